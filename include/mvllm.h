@@ -470,14 +470,17 @@ int mv_graph_destroy(void* graph_exec);
 int mv_linear_any(const void* x, int64_t ldx, const void* w, int64_t ldw, float* y, int64_t ldy, int m, int n,
                   int k, int f32, mv_stream_t stream);
 
-/* x[r,:] = table[ids[r],:] * scale (fp32), h = the same in the activation type. */
+/* x[r,:] = table[ids[r],:] * scale (fp32), h = the same in the activation type; norm_w != NULL:
+ * h = act( x / sqrt(mean(x^2) + eps) * (offset + norm_w) ). */
 int mv_embed_scaled(const void* table, const int32_t* ids, float* x, int64_t ldx, void* h, int64_t ldh, int rows,
-                    int n, int vocab, float scale, int f32, mv_stream_t stream);
+                    int n, int vocab, float scale, const float* norm_w, float eps, float offset, int f32,
+                    mv_stream_t stream);
 
-/* v = s1*y1 (+ s2*y2 when y2 != NULL); x += v / sqrt(mean(v^2) + eps) * (1 + w); h = act(x). */
+/* v = s1*y1 (+ s2*y2 when y2 != NULL) (+ bias [n]); x += mult * v / sqrt(mean(v^2) + eps) * (1 + w); h = act(x), or
+ * with next_w != NULL the next sublayer's norm of the new x, h = act( x / sqrt(mean(x^2) + eps) * (1 + next_w) ). */
 int mv_postnorm_residual(const float* y1, int64_t ld1, const float* y2, int64_t ld2, float s1, float s2,
-                         const float* w, float eps, float* x, int64_t ldx, void* h, int64_t ldh, int rows, int n,
-                         int f32, mv_stream_t stream);
+                         const float* bias, const float* w, float eps, float mult, const float* next_w, float* x,
+                         int64_t ldx, void* h, int64_t ldh, int rows, int n, int f32, mv_stream_t stream);
 
 /* out[r,:] = act( x[idx[r],:] / sqrt(mean(.^2) + eps) * (1 + w) ); idx == NULL: row r itself. */
 int mv_offset_rmsnorm_gather(const float* x, int64_t ldx, const int32_t* idx, const float* w, float eps, void* out,
@@ -536,10 +539,11 @@ int mv_scan_chunked(const float* q, int64_t ldq, int q_div, const float* k, int6
 int mv_rotary_pairs(float* x, int64_t ld, const double* inv_freq, const int32_t* tok_pos, int tokens, int heads,
                     int dim, int rot, float scale, mv_stream_t stream);
 
-/* Rows cut into `groups` equal parts, each divided by its root mean square; gate_first: the part is
- * y * silu(gate) before that, else silu(gate) multiplies after; w (fp32 [n]) multiplies last or is NULL. */
+/* Rows cut into `groups` equal parts, each divided by its root mean square; mode 1: the part is
+ * y * silu(gate) before that; mode 0: silu(gate), mode 2: sigmoid(gate) multiplies after; w (fp32 [n], or [n / groups]
+ * for all parts alike when w_shared) multiplies last or is NULL. */
 int mv_gated_group_norm(const float* y, int64_t ldy, const float* gate, int64_t ldg, const float* w, void* out,
-                        int64_t ldo, int rows, int n, int groups, int gate_first, float eps, int f32,
+                        int64_t ldo, int rows, int n, int groups, int mode, int w_shared, float eps, int f32,
                         mv_stream_t stream);
 
 /* Rows of qkv are [heads x d | kv_heads x d | kv_heads x dv] fp32.  Queries are divided by their root
@@ -569,7 +573,8 @@ int mv_qk_rotary_store(float* qk, int64_t ld, const float* q_bias, const float* 
  * run one workgroup per (token, key/value head, up to eight of its query heads, split of the keys) - every key and value
  * is read once for those heads - and, with splits > 1, a second launch merges the splits' pieces.
  * short_tokens: how many of the step's tokens lie in rows of up to max_len tokens (-1: not known); 0 lets a step whose
- * rows all went to the tiled kernel skip the launch of the per-token form.  With a chunk table (chunks > 0:
+ * rows all went to the tiled kernel skip the launch of the per-token form.  gate != NULL (fp32 [tokens, heads * dv]):
+ * out is multiplied by sigmoid(gate) before it is rounded.  With a chunk table (chunks > 0:
  * rows of more than max_len tokens cut into runs of up to 64, as for mv_scan_chunked; row_len per row), bf16
  * and a head shape the tiled kernel is built for - (d, dv) in (32,32) (64,64) (96,96) (128,128) (128,64)
  * (64,128), 64-token pages - those rows run on the matrix cores, a workgroup per (chunk, head): q.k in bf16
@@ -580,7 +585,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
                    int page, const float* slopes, int tokens, int heads, int kv_heads, int d, int dv, float scale,
                    int window, int f32, const int32_t* row_len, const int32_t* ch_start, const int32_t* ch_len,
                    int chunks, int max_len, int keep_first, const float* sinks, float* part, int splits,
-                   int short_tokens, mv_stream_t stream);
+                   int short_tokens, const float* gate, int64_t ldg, mv_stream_t stream);
 /* How many splits of the keys mv_window_attn should be given for a step of `tokens` tokens (1: none). */
 int mv_window_attn_splits(int tokens, int heads, int kv_heads, int window, int keep_first);
 
@@ -759,6 +764,49 @@ int mv_diff_attn(const float* q, int64_t ldq, const void* k_cache, const void* v
                  float scale, float cap, float lambda, float out_scale, float eps, int f32, const int32_t* row_len,
                  const int32_t* ch_start, const int32_t* ch_len, int chunks, int max_len, int short_tokens,
                  mv_stream_t stream);
+
+/* ---- norm over whole projections, mixed values (seq_mix.hip) --------------------------------------------- */
+
+/* Rows of qkv: q [heads * d] | k [kv_heads * d] | v [kv_heads * dv] of one projection (fp32).  q and k: + bias, RMS norm
+ * over ALL heads at once (q_norm [heads * d], k_norm [kv_heads * d], plain weights; NULL: no norm), rotation of each
+ * head's first `rot` dimensions by position * inv_freq[i] (fp64 [rot / 2]; adjacent pairs, or i with i + rot / 2); q in
+ * place, k to k_cache [pages, page, kv_heads, d].  v: + bias; mix 1: kept in v_first [T, kv_heads * dv]; mix 2:
+ * v = (1 - lam) v + lam v_first; to v_cache.  Biases may be NULL. */
+int mv_qkv_norm_rotary_store(float* qkv, int64_t ld, const float* q_bias, const float* k_bias, const float* v_bias,
+                             const float* q_norm, const float* k_norm, float eps, const double* inv_freq,
+                             float* v_first, int mix, float lam, void* k_cache, void* v_cache, const int32_t* tok_row,
+                             const int32_t* tok_pos, const int32_t* block_table, int bt_stride, int page, int tokens,
+                             int heads, int kv_heads, int d, int dv, int rot, int adjacent, int f32,
+                             mv_stream_t stream);
+
+/* ---- delta-rule memory with a decay per state row (delta.hip) ------------------------------------------------- */
+
+/* proj [T, ldp]: q [kv_heads * n] | k [kv_heads * n] | v [heads * p], then `heads` logits at b_off and low_n columns
+ * at low_off.  out [T, ldo] = silu of a causal convolution per channel (wt [taps, C] fp32, last row = the current
+ * token; inputs before the step from state [slots, taps - 1, C], zeros when row_ctx == 0, which then keeps each row's
+ * last taps - 1 inputs); every head of q and k divided by sqrt(sum of squares + eps), q times q_scale as well.
+ * beta [T, heads] = sigmoid(logits); low [T, ldl] = the low_n columns in the activation type.  n <= 512. */
+int mv_delta_prep(const float* proj, int64_t ldp, int b_off, int low_off, int low_n, float* state, const float* wt,
+                  float* out, int64_t ldo, float* beta, void* low, int64_t ldl, const int32_t* tok_row,
+                  const int32_t* row_start, const int32_t* row_len, const int32_t* row_ctx, const int32_t* row_slot,
+                  int tokens, int rows, int kv_heads, int n, int heads, int p, int taps, float eps, float q_scale,
+                  int f32, mv_stream_t stream);
+/* Per head (head h reads q and k of head h / (heads / kv_heads)), S [n, p] in state [slots, heads, n, p] fp32 (zero when
+ * row_ctx == 0):  g = exp(-exp(a_log[h]) softplus(gate_in + dt_bias)) per state row;  S = diag(g) S;
+ * u = beta (v - S^T k);  S += k u^T;  o = S^T q;  out = act( o / sqrt(mean(o^2) + eps) * norm * sigmoid(z) ).
+ * qkv as mv_delta_prep leaves it, gate_in [T, heads * n], z [T, heads * p], norm [p].  p <= 256, and n such that a
+ * thread of 1024 holds at most 64 state values of its column (n <= 256 at p = 256, twice that at half the width).
+ * chunks > 0 (mv_delta_chunked_ok(n, p)): rows of more than max_len tokens run in chunks of 64 (tables as for
+ * mv_scan_chunked; scratch: chunks * heads * mv_delta_scratch_floats(n, p) fp32 values); short_tokens: tokens in
+ * the other rows (-1: unknown). */
+int mv_delta_rule(const float* qkv, int64_t ldq, const float* gate_in, int64_t lda, const float* z, int64_t ldz,
+                  const float* beta, const float* dt_bias, const float* a_log, const float* norm, float* state,
+                  void* out, int64_t ldo, const int32_t* row_start, const int32_t* row_len, const int32_t* row_ctx,
+                  const int32_t* row_slot, int rows, int kv_heads, int heads, int n, int p, float eps, float* scratch,
+                  const int32_t* ch_start, const int32_t* ch_len, const int32_t* row_ch0, const int32_t* row_nch,
+                  int chunks, int max_len, int short_tokens, int f32, mv_stream_t stream);
+int mv_delta_chunked_ok(int n, int p);
+int64_t mv_delta_scratch_floats(int n, int p);
 
 #ifdef __cplusplus
 }

@@ -92,8 +92,8 @@ PROTOTYPES = {
     "mv_allgather_rows": (_I, [_P, _P, _L, _P, _L, _I, _I, _P]),
     "mv_allreduce_addnorm": (_I, [_P, _P, _L, _P, _I, _P, _L, _P, _L, _P, _F, _P, _L, _I, _I, _I, _P]),
     "mv_linear_any": (_I, [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _P]),
-    "mv_embed_scaled": (_I, [_P, _P, _P, _L, _P, _L, _I, _I, _I, _F, _I, _P]),
-    "mv_postnorm_residual": (_I, [_P, _L, _P, _L, _F, _F, _P, _F, _P, _L, _P, _L, _I, _I, _I, _P]),
+    "mv_embed_scaled": (_I, [_P, _P, _P, _L, _P, _L, _I, _I, _I, _F, _P, _F, _F, _I, _P]),
+    "mv_postnorm_residual": (_I, [_P, _L, _P, _L, _F, _F, _P, _P, _F, _F, _P, _P, _L, _P, _L, _I, _I, _I, _P]),
     "mv_offset_rmsnorm_gather": (_I, [_P, _L, _P, _P, _F, _P, _L, _I, _I, _I, _P]),
     "mv_relu_squared": (_I, [_P, _L, _P, _L, _I, _I, _I, _P]),
     "mv_softcap": (_I, [_P, _L, _F, _P]),
@@ -105,10 +105,10 @@ PROTOTYPES = {
     "mv_scan_chunked": (_I, [_P, _L, _I, _P, _L, _I, _P, _L, _P, _L, _P, _L, _P, _P, _P, _L, _P, _P, _P,
                              _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P]),
     "mv_rotary_pairs": (_I, [_P, _L, _P, _P, _I, _I, _I, _I, _F, _P]),
-    "mv_gated_group_norm": (_I, [_P, _L, _P, _L, _P, _P, _L, _I, _I, _I, _I, _F, _I, _P]),
+    "mv_gated_group_norm": (_I, [_P, _L, _P, _L, _P, _P, _L, _I, _I, _I, _I, _I, _F, _I, _P]),
     "mv_qk_unitnorm_store": (_I, [_P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P]),
     "mv_window_attn": (_I, [_P, _L, _P, _P, _P, _L, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _F, _I, _I,
-                            _P, _P, _P, _I, _I, _I, _P, _P, _I, _I, _P]),
+                            _P, _P, _P, _I, _I, _I, _P, _P, _I, _I, _P, _L, _P]),
     "mv_window_attn_splits": (_I, [_I, _I, _I, _I, _I]),
     "mv_qk_rotary_store": (_I, [_P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _L, _P, _L,
                                 _I, _I, _F, _F, _I, _P]),
@@ -149,6 +149,14 @@ PROTOTYPES = {
                                _I, _I, _I, _P]),
     "mv_diff_attn": (_I, [_P, _L, _P, _P, _P, _L, _P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _F, _F,
                           _I, _P, _P, _P, _I, _I, _I, _P]),
+    "mv_qkv_norm_rotary_store": (_I, [_P, _L, _P, _P, _P, _P, _P, _F, _P, _P, _I, _F, _P, _P, _P, _P, _P, _I, _I, _I, _I,
+                                      _I, _I, _I, _I, _I, _I, _P]),
+    "mv_delta_prep": (_I, [_P, _L, _I, _I, _I, _P, _P, _P, _L, _P, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I,
+                           _F, _F, _I, _P]),
+    "mv_delta_rule": (_I, [_P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P,
+                           _P, _P, _P, _P, _I, _I, _I, _I, _P]),
+    "mv_delta_chunked_ok": (_I, [_I, _I]),
+    "mv_delta_scratch_floats": (_L, [_I, _I]),
     "mv_graph_begin_capture": (_I, [_P]),
     "mv_graph_end_capture": (_I, [_P, ctypes.POINTER(c_void_p)]),
     "mv_graph_launch": (_I, [_P, _P]),

@@ -65,6 +65,18 @@ Per layer (Solopel; pre-norm, every sublayer output passes a sigmoid gate comput
             products scaled by the pair's score (the score scales the expert's input) -> down by segment; shared
             expert's gate|up|R2 in one projection; plain sum
   loop      a pass of the looped span starts from W_in [x | x0] + step_t, x0 the embedding
+
+Per layer (Dugazen; an RMS norm with weight 1 + w in front of every sublayer and another on its output):
+  residual  x += m * norm(y + bias) of the sublayer before and the next sublayer's norm of the new x, in one launch (the
+            last one hands out the final norm where every token's logits are wanted)
+  delta     ONE projection gives q | k | v | head logits | low-rank columns -> short convolutions with SiLU (inputs kept
+            per slot), unit length of q and k, beta, the low-rank columns cast, in one launch -> one product with the
+            block-diagonal [W_a2, W_g2] gives gate inputs and output-gate logits -> decay gates, delta rule (state per
+            slot), unit-RMS per head, weight, sigmoid gate -> out-projection
+  attention ONE projection gives q | k | v | gate -> biases, norm over the whole of q and of k, rotation, values mixed
+            with the first mixing layer's, keys and values into the pages, in one launch -> windowed softmax attention
+            with the sigmoid gate on its output -> out-projection
+  dense     gate|up projection -> clamped gate -> down
 """
 import logging
 import math
@@ -73,6 +85,7 @@ from typing import Dict, List, Optional
 import torch
 
 from ...kernel import ragged_ops as ops
+from ...models import dugazen
 from ...models.nesisun import GATE_SLOPE, WEIGHT_SUM_FLOOR
 from ...models.pagazen import mamba2_sizes
 from ..state_cache import HybridCacheManager, RaggedStep
@@ -108,6 +121,7 @@ class RaggedRunner:
         self.sandwich = cfg.architecture == "Fagunex"     # Dynamic Tanh before and after each sublayer
         self.parallel_prenorm = cfg.architecture == "Nesisun"   # one RMS norm feeds mixer and feed-forward alike
         self.gated_prenorm = cfg.architecture == "Solopel"      # pre-norm layers whose sublayer outputs pass a gate
+        self.double_norm = cfg.architecture == "Dugazen"        # an RMS norm in front of every sublayer and one behind it
         for wi, layer in self.runs:
             if wi not in self._w:
                 self._w[wi] = self._prepare_layer(wi, layer)
@@ -145,6 +159,13 @@ class RaggedRunner:
         g = self.model.get
         return (self._small(g(name)), self._small(g(name + ".b")), self._small(g(name + ".alpha")).reshape(1))
 
+    def _linear_padded(self, *parts, multiple: int = 16):
+        """The parts as one projection, zero rows filling its width up to what the wave-tile projections take."""
+        pad = -sum(p.shape[0] for p in parts) % multiple
+        if pad:
+            parts = parts + (torch.zeros(pad, parts[0].shape[1], dtype=parts[0].dtype),)
+        return self._linear(*parts)
+
     def _stacked(self, parts):
         """[E, n, k] in the activation type: the same projection of several experts or heads."""
         w = torch.stack([self._act(p) for p in parts], dim=0).contiguous()
@@ -158,6 +179,8 @@ class RaggedRunner:
             return self._prepare_nesisun(i, layer)
         if self.gated_prenorm:
             return self._prepare_solopel(i, layer)
+        if self.double_norm:
+            return self._prepare_dugazen(i, layer)
         g, p, m = self.model.get, f"l{i}.", layer["mixer"]
         w = {"norm1": self._small(g(p + "norm1"))}
         if layer["type"] == "mamba2":
@@ -296,6 +319,41 @@ class RaggedRunner:
                     w.update(rg2=self._linear(g(p + "rg2")))
         return w
 
+    def _prepare_dugazen(self, i: int, layer: dict) -> dict:
+        g, p, m, W = self.model.get, f"l{i}.", layer["mixer"], self.width
+        w = {"norm1": self._small(g(p + "norm1")), "norm1b": self._small(g(p + "norm1b"))}
+        H, G, d, dv = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
+        if layer["type"] == "attention":
+            rot = int(m["rot"]["dims"])
+            inv_freq = float(m["rot"]["base"]) ** (-2.0 * torch.arange(max(rot // 2, 1), dtype=torch.float64) / max(rot, 1))
+            w.update(w_in=self._linear_padded(g(p + "mix.q"), g(p + "mix.k"), g(p + "mix.v"), g(p + "mix.g")),
+                     w_o=self._linear(g(p + "mix.o")), inv_freq=inv_freq.to(self.device),
+                     mix=0 if not m.get("v_mix") else (1 if i == self.cfg.first_value_mix() else 2))
+            w.update({k: self._small(g(p + "mix." + n)) for k, n in (
+                ("q_b", "q.b"), ("k_b", "k.b"), ("v_b", "v.b"), ("o_b", "o.b"), ("q_norm", "q.norm"), ("k_norm", "k.norm"))})
+            w["lam"] = float(g(p + "mix.vmix").float()) if w["mix"] == 2 else 0.0
+        else:
+            a1, g1, a2, g2 = (g(p + "mix." + n) for n in ("a1", "g1", "a2", "g2"))
+            C, ra, rg = 2 * G * d + H * dv, a1.shape[0], g1.shape[0]
+            rows = lambda n: torch.zeros(n, W, dtype=a1.dtype)   # noqa: E731
+            # [q | k | v | head logits (| zeros) | a1 | g1 (| zeros)]; the second maps of both low-rank pairs are one
+            # block-diagonal product over the a1 | g1 columns
+            low = -(-(ra + rg) // 64) * 64
+            second = torch.zeros(H * (d + dv), low, dtype=a1.dtype)
+            second[:H * d, :ra], second[H * d:, ra:ra + rg] = a2, g2
+            b_pad = -(C + H) % 16
+            w.update(w_in=self._linear(g(p + "mix.q"), g(p + "mix.k"), g(p + "mix.v"), g(p + "mix.b"), rows(b_pad), a1, g1,
+                                       rows(low - ra - rg)),
+                     low_off=C + H + b_pad, low=low, w_second=self._linear(second), w_o=self._linear(g(p + "mix.o")),
+                     conv=self._small(torch.cat([g(p + "mix.q.conv"), g(p + "mix.k.conv"), g(p + "mix.v.conv")], dim=0).t()),
+                     a_log=self._small(g(p + "mix.A_log")), dt_bias=self._small(g(p + "mix.dt_bias")),
+                     norm=self._small(g(p + "mix.norm")))
+        mlp = layer.get("mlp")
+        if mlp:
+            w.update(norm2=self._small(g(p + "norm2")), norm2b=self._small(g(p + "norm2b")),
+                     gate_up=self._linear(g(p + "mlp.gate"), g(p + "mlp.up")), down=self._linear(g(p + "mlp.down")))
+        return w
+
     # ------------------------------------------------------------------ cache geometry
     def cache_layout(self):
         """(kv_layers, state_layers) for HybridCacheManager: what every layer RUN keeps per sequence."""
@@ -311,6 +369,15 @@ class RaggedRunner:
                     kv[i] = (G, 2 * d, dv)                     # both maps' keys of a key/value head side by side
                     if int(m.get("conv") or 0) > 1:
                         state[i]["qkv"] = (int(m["conv"]) - 1, H * 2 * d + G * 2 * d + G * dv)
+            return kv, state
+        if self.cfg.architecture == "Dugazen":
+            for i, (_, layer) in enumerate(self.runs):
+                m = layer["mixer"]
+                H, G, d, dv = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
+                if layer["type"] == "attention":
+                    kv[i] = (G, d, dv)
+                else:      # the convolutions' last inputs and the memory itself
+                    state[i] = {"conv": (int(m["conv"]) - 1, 2 * G * d + H * dv), "delta": (H, d, dv)}
             return kv, state
         for i, (_, layer) in enumerate(self.runs):
             m = layer["mixer"]
@@ -439,13 +506,12 @@ class RaggedRunner:
         B, slots = step.rows, list(step.slots)
         idx = torch.tensor(slots, dtype=torch.long, device=self.device)
         saved = [(t, t.index_select(0, idx)) for named in cache.states.values() for t in named.values()]
-        all_rows = torch.arange(B, dtype=torch.int32, device=self.device)
         side = torch.cuda.Stream(device=self.device)
         side.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(side):
             self._arena, self._measured = None, 0
             try:
-                self._run(step, cache, all_rows, None)
+                self._run(step, cache, None, None)
             finally:   # whatever that run did to the slots' state is undone: the step itself is still to come
                 for t, old in saved:
                     t.index_copy_(0, idx, old)
@@ -454,7 +520,7 @@ class RaggedRunner:
             self._arena, self._arena_off = arena, 0
             nv.check("mv_graph_begin_capture", nv.lib().mv_graph_begin_capture(side.cuda_stream))
             try:
-                logits = self._run(step, cache, all_rows, None)
+                logits = self._run(step, cache, None, None)
             finally:
                 handle = ctypes.c_void_p()
                 rc = nv.lib().mv_graph_end_capture(side.cuda_stream, ctypes.byref(handle))
@@ -462,10 +528,11 @@ class RaggedRunner:
             nv.check("mv_graph_end_capture", rc)
         torch.cuda.current_stream().wait_stream(side)
         logger.info("captured a decoding step of %d rows (%d KiB of intermediates)", B, arena.numel() >> 10)
-        return HipGraph(handle), arena, logits, all_rows      # the arena and the row list stay alive with the graph
+        return HipGraph(handle), arena, logits      # the arena stays alive with the graph
 
     def _run(self, step: RaggedStep, cache: HybridCacheManager, want, residuals) -> torch.Tensor:
         cfg, T = self.cfg, step.tokens
+        normed = None
         if not self.gated_prenorm:       # that design's stack lays out its own streams
             x, h = self._f32buf(T, self.width), self._actbuf(T, self.width)
         if self.parallel_prenorm:
@@ -480,6 +547,11 @@ class RaggedRunner:
                     residuals.append(x.clone())
         elif self.gated_prenorm:
             x = self._solopel_stack(step, cache, residuals)
+        elif self.double_norm:
+            # where every token's logits are wanted the last residual step hands out the final norm as well
+            if want is None:
+                normed = self._actbuf(T, self.width)
+            self._dugazen_stack(step, cache, residuals, x, h, normed)
         elif self.sandwich:
             ops.embed_scaled(self.embed, step.ids, 1.0, x, h)
             for li, (wi, layer) in enumerate(self.runs):
@@ -505,10 +577,14 @@ class RaggedRunner:
                 if residuals is not None:
                     residuals.append(x.clone())
         rows = T if want is None else want.numel()
-        normed = self._actbuf(rows, self.width)
         if rows == 0:
             return self._f32buf(0, self.vocab_size)
-        if self.sandwich:
+        have = normed is not None
+        if not have:
+            normed = self._actbuf(rows, self.width)
+        if have:
+            pass
+        elif self.sandwich:
             ops.dyt_gather(x, want, self.final_norm, normed)
         elif self.parallel_prenorm:
             ops.rmsnorm_gather(x, want, self.final_norm, cfg.eps, normed)
@@ -681,6 +757,70 @@ class RaggedRunner:
         diff = float(m["diff"])
         ops.diff_attn(q, kc, vc, a, proj[:, C:C + H], step, H, G, d, dv, float(m["scale"]), float(m.get("softcap") or 0.0),
                       w["lam"], 1.0 - diff, self.cfg.eps, tiled=self.tiled_attn)
+        return w["w_o"](a, self._f32buf(T, self.width))
+
+    # ------------------------------------------------------------------ Dugazen layers
+    def _dugazen_stack(self, step: RaggedStep, cache: HybridCacheManager, residuals, x, h, normed):
+        """All layers on the stream x (fp32, updated in place); h is scratch of the activation type; `normed` (optional)
+        receives the final norm of the stream."""
+        cfg, T = self.cfg, step.tokens
+        eps, mult = cfg.eps, cfg.residual_mult
+        first = self._w[self.runs[0][0]]["norm1"]
+        ops.embed_scaled(self.embed, step.ids, 1.0, x, h, w=first, eps=eps, offset=1.0)
+        v_first = None
+        for li, (wi, layer) in enumerate(self.runs):
+            w, mlp = self._w[wi], layer.get("mlp")
+            if layer["type"] == "attention":
+                if w["mix"] == 1:
+                    v_first = self._f32buf(T, int(layer["mixer"]["kv_heads"]) * int(layer["mixer"]["vdim"]))
+                y, bias = self._dugazen_attention(li, w, layer["mixer"], h, step, cache, v_first), w["o_b"]
+            else:
+                y, bias = self._channel_delta(li, w, layer["mixer"], h, step, cache), None
+            last = li + 1 == len(self.runs)
+            nxt, out = (self.final_norm, normed) if last else (self._w[self.runs[li + 1][0]]["norm1"], h)
+            if last and normed is None:
+                nxt, out = None, h
+            if mlp:
+                ops.postnorm_residual(y, w["norm1b"], eps, x, h, bias=bias, mult=mult, next_w=w["norm2"])
+                ff = int(mlp["ff"])
+                act = self._actbuf(T, ff)
+                ops.gated_act(w["gate_up"](h, self._f32buf(T, 2 * ff)), act, ops.GATE_CLAMPED, float(mlp["limit"]),
+                              dugazen.GATE_SLOPE)
+                y, bias = w["down"](act, self._f32buf(T, self.width)), None
+                ops.postnorm_residual(y, w["norm2b"], eps, x, out, mult=mult, next_w=nxt)
+            else:
+                ops.postnorm_residual(y, w["norm1b"], eps, x, out, bias=bias, mult=mult, next_w=nxt)
+            if residuals is not None:
+                residuals.append(x.clone())
+
+    def _channel_delta(self, li, w, m, h, step: RaggedStep, cache: HybridCacheManager):
+        T, st = step.tokens, cache.states[li]
+        H, K, n, p = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
+        C = 2 * K * n + H * p
+        proj = w["w_in"](h, self._f32buf(T, w["w_in"].n))            # [q | k | v | head logits | low-rank columns]
+        qkv, beta, low = self._f32buf(T, C), self._f32buf(T, H), self._actbuf(T, w["low"])
+        ops.delta_prep(proj, st["conv"], w["conv"], qkv, beta, low, step, K, n, H, p, C, w["low_off"], dugazen.UNIT_EPS)
+        gates = w["w_second"](low, self._f32buf(T, H * (n + p)))     # [decay gate inputs | output gate logits]
+        u = self._actbuf(T, H * p)
+        ops.delta_rule(qkv, gates[:, :H * n], gates[:, H * n:], beta, w["dt_bias"], w["a_log"], w["norm"], st["delta"], u,
+                       step, K, H, n, p, self.cfg.eps, chunked=self.chunked_scan)
+        return w["w_o"](u, self._f32buf(T, self.width))
+
+    def _dugazen_attention(self, li, w, m, h, step: RaggedStep, cache: HybridCacheManager, v_first):
+        T = step.tokens
+        H, G, d, dv = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
+        C = (H + G) * d + G * dv
+        proj = w["w_in"](h, self._f32buf(T, w["w_in"].n))            # [q | k | v | output gate (| zeros)]
+        kc, vc = cache.k_caches[li], cache.v_caches[li]
+        ops.qkv_norm_rotary_store(proj[:, :C], kc, vc, step, H, G, d, dv, w["inv_freq"], int(m["rot"]["dims"]), self.cfg.eps,
+                                  q_bias=w["q_b"], k_bias=w["k_b"], v_bias=w["v_b"], q_norm=w["q_norm"],
+                                  k_norm=w["k_norm"], v_first=v_first, mix=w["mix"], lam=w["lam"])
+        a = self._actbuf(T, H * dv)
+        window = int(m["mask"]["size"])
+        splits = ops.window_attn_splits(T, H, G, window) if self.grouped_attn else 0
+        part = self._f32buf(1, T * H * splits * (dv + 2)) if splits else None
+        ops.window_attn(proj[:, :H * d], kc, vc, a, step, None, H, G, d, dv, float(m["scale"]), window,
+                        tiled=self.tiled_attn, part=part, splits=splits, gate=proj[:, C:C + H * dv])
         return w["w_o"](a, self._f32buf(T, self.width))
 
     # ------------------------------------------------------------------ Fagunex layers

@@ -1,0 +1,770 @@
+// Delta-rule memory with a decay per state row, over a ragged step (rows of tokens back to back, as in seq_mix.hip).
+// Per head, with S [n, p] kept per sequence in its state slot:
+//   S <- diag(g_t) S;   u_t = beta_t (v_t - S^T k_t);   S <- S + k_t u_t^T;   o_t = S^T q_t
+// g_t in (0, 1)^n, q and k unit vectors that a group of heads may share.
+//
+//   delta_prep     the short convolutions with SiLU over the q | k | v columns of one projection, unit length per
+//                  head of q and k, beta = sigmoid, and the low-rank inputs of the gates in the activation type
+//   delta_rule     rows of few tokens: one workgroup per (row, head) with S in registers, token by token; rows of
+//                  many tokens: chunks of 64 (below).  Both form the gates g = exp(-exp(A) softplus(a + bias)) and
+//                  hand out act( o / rms(o) * w * sigmoid(z) )
+// All of it in fp32; only what goes to a projection is of the activation type.
+#include "common.h"
+
+namespace mv {
+
+template <bool F32> struct ActD;
+template <> struct ActD<true> {
+    typedef float T;
+    static __device__ __forceinline__ void st(float* p, float v) { *p = v; }
+};
+template <> struct ActD<false> {
+    typedef uint16_t T;
+    static __device__ __forceinline__ void st(uint16_t* p, float v) { *p = (uint16_t)f32_to_bf16_bits(v); }
+};
+
+__device__ __forceinline__ float sigmoid_d(float v) { return 1.0f / (1.0f + expf(-v)); }
+
+struct DeltaRows {
+    const int *tok_row, *row_start, *row_len, *row_ctx, *row_slot;
+};
+
+constexpr int kDeltaMaxTaps = 16;
+constexpr int kDeltaMaxN = 512;     // state rows per head
+
+struct DeltaPrepArgs {
+    const float* proj;      // [T, ldp]: q [K n] | k [K n] | v [H p] at 0, beta logits at b_off, low-rank columns at low_off
+    int64_t ldp, ldo, ldl;
+    int b_off, low_off, low_n;
+    float* state;           // [slots, taps - 1, C]
+    const float* wt;        // [taps, C]
+    float* out;             // [T, C]
+    float* beta;            // [T, H]
+    void* low;              // [T, low_n] activation type
+    DeltaRows r;
+    int T, K, n, H, p, taps, in_place;
+    float eps, qscale;
+};
+
+// One wave per (token, unit): a head of q, a head of k, 256 channels of v, or the betas with the low-rank columns.
+// in_place: every row has one token, so the wave that reads a channel's kept inputs also moves them on.
+template <bool F32>
+__global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a) {
+    const int lane = threadIdx.x & 63;
+    const int vu = (a.H * a.p + 255) / 256, units = 2 * a.K + vu + 1;
+    const int unit = blockIdx.y;                                    // the four waves of a workgroup: neighbouring tokens
+    const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t >= a.T) return;
+    const float* row = a.proj + (int64_t)t * a.ldp;
+    if (unit == units - 1) {
+        for (int h = lane; h < a.H; h += 64) a.beta[(int64_t)t * a.H + h] = sigmoid_d(row[a.b_off + h]);
+        typename ActD<F32>::T* lo = (typename ActD<F32>::T*)a.low + (int64_t)t * a.ldl;
+        for (int c = lane; c < a.low_n; c += 64) ActD<F32>::st(lo + c, row[a.low_off + c]);
+        return;
+    }
+    const bool head = unit < 2 * a.K;
+    const int C = 2 * a.K * a.n + a.H * a.p;
+    const int c0 = head ? unit * a.n : 2 * a.K * a.n + (unit - 2 * a.K) * 256;
+    const int cnt = head ? a.n : (C - c0 < 256 ? C - c0 : 256);
+    const int b = a.r.tok_row[t], rel = t - a.r.row_start[b], keep = a.taps - 1;
+    const bool carried = a.r.row_ctx[b] > 0;
+    float* st = a.state + (int64_t)a.r.row_slot[b] * keep * C;
+    float y[kDeltaMaxN / 64];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < kDeltaMaxN / 64; ++i) {
+        y[i] = 0.f;
+        if (64 * i >= cnt) continue;
+        const int cl = lane + 64 * i;
+        if (cl >= cnt) continue;
+        const int c = c0 + cl;
+        float acc = 0.f;
+        for (int j = 0; j < a.taps; ++j) {
+            const int src = rel - keep + j;
+            float v;
+            if (src >= 0) v = row[(int64_t)(j - keep) * a.ldp + c];
+            else v = carried ? st[(int64_t)(src + keep) * C + c] : 0.f;
+            acc = fmaf(a.wt[(int64_t)j * C + c], v, acc);
+            // the channel's kept inputs move on by one (tap j of this token is tap j - 1 of the next)
+            if (a.in_place && j > 0) st[(int64_t)(j - 1) * C + c] = v;
+        }
+        y[i] = acc * sigmoid_d(acc);
+        ss += y[i] * y[i];
+    }
+    float f = 1.0f;
+    if (head) f = (1.0f / sqrtf(wave_sum(ss) + a.eps)) * (unit < a.K ? a.qscale : 1.0f);
+#pragma unroll
+    for (int i = 0; i < kDeltaMaxN / 64; ++i) {
+        const int cl = lane + 64 * i;
+        if (cl < cnt) a.out[(int64_t)t * a.ldo + c0 + cl] = y[i] * f;
+    }
+}
+
+// keeps each row's last taps - 1 inputs (rows of any length; used when some row has more than one token)
+__global__ __launch_bounds__(256) void delta_conv_state_kernel(DeltaPrepArgs a, int B) {
+    const int C = 2 * a.K * a.n + a.H * a.p, keep = a.taps - 1;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= (int64_t)B * C) return;
+    const int b = (int)(i / C), c = (int)(i % C);
+    const int len = a.r.row_len[b], start = a.r.row_start[b];
+    const bool carried = a.r.row_ctx[b] > 0;
+    float* st = a.state + (int64_t)a.r.row_slot[b] * keep * C + c;
+    float old[kDeltaMaxTaps];
+    for (int s = 0; s < keep; ++s) old[s] = carried ? st[(int64_t)s * C] : 0.f;
+    for (int s = 0; s < keep; ++s) {
+        const int rel = len - keep + s;
+        st[(int64_t)s * C] = rel >= 0 ? a.proj[(int64_t)(start + rel) * a.ldp + c] : old[s + len];
+    }
+}
+
+struct DeltaArgs {
+    const float* qkv;       // [T, ldq]: q [K n] | k [K n] | v [H p], as delta_prep leaves them
+    const float* a;         // [T, lda]: raw gate inputs [H n]
+    const float* z;         // [T, ldz]: logits of the output gate [H p]
+    const float *beta, *dt_bias, *a_log, *norm;
+    int64_t ldq, lda, ldz, ldo;
+    float* state;           // [slots, H, n, p]
+    void* out;              // [T, ldo] activation type
+    DeltaRows r;
+    int K, H, n, p, max_len;
+    float eps;
+    // chunks of long rows
+    const int *ch_start, *ch_len, *row_ch0, *row_nch;
+    float *qd, *wk, *kt, *uv, *bm, *s0, *gc;     // scratch, see DeltaScratch
+};
+
+__device__ __forceinline__ float decay_gate(float raw, float bias, float neg_a) {
+    const float v = raw + bias;
+    const float sp = fmaxf(v, 0.f) + log1pf(expf(-fabsf(v)));     // log(1 + e^v)
+    return expf(neg_a * sp);
+}
+
+// One workgroup per (head, row).  Thread (ng, cl) holds the state rows ng * npt .. + npt of column cl; columns are
+// padded to `pw`, a power of two.  The two sums over state rows (what the key reads, what the query reads) are formed in one
+// pass over the decayed state; the write's share of the read-out is u (k . q).
+template <bool F32, int MAXN>
+__global__ void delta_scan_kernel(DeltaArgs a, int pw) {
+    extern __shared__ float lds[];
+    const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, NT = blockDim.x;
+    const int len = a.r.row_len[b], start = a.r.row_start[b];
+    if (a.max_len > 0 && len > a.max_len) return;      // the chunked form's rows; the whole workgroup
+    const int NG = NT / pw, cl = tid & (pw - 1), ng = tid / pw;
+    const int n = a.n, p = a.p, npt = (n + NG - 1) / NG, n0 = ng * npt;
+    float* qs = lds;
+    float* ks = qs + n;
+    float* gs = ks + n;
+    float* pk = gs + n;             // [NG][pw]
+    float* pq = pk + NT;            // [NG][pw]
+    float* pd = pq + NT;            // [NG] partial sums of k . q
+    float* red = pd + NG;           // [pw / 64]
+    const bool vc = cl < p;
+    const int kh = h / (a.H / a.K);
+    const bool carried = a.r.row_ctx[b] > 0;
+    float* sp = a.state + (((int64_t)a.r.row_slot[b] * a.H + h) * n + n0) * p + cl;
+    float S[MAXN];
+#pragma unroll
+    for (int i = 0; i < MAXN; ++i) S[i] = (carried && vc && i < npt && n0 + i < n) ? sp[(int64_t)i * p] : 0.f;
+    const float neg_a = -expf(a.a_log[h]);
+    const float wn = vc ? a.norm[cl] : 0.f;
+    for (int t = 0; t < len; ++t) {
+        const int64_t tok = start + t;
+        const float* qp = a.qkv + tok * a.ldq + (int64_t)kh * n;
+        const float* kp = qp + (int64_t)a.K * n;
+        for (int i = tid; i < n; i += NT) {
+            qs[i] = qp[i];
+            ks[i] = kp[i];
+            gs[i] = decay_gate(a.a[tok * a.lda + (int64_t)h * n + i], a.dt_bias[(int64_t)h * n + i], neg_a);
+        }
+        const float vv = vc ? a.qkv[tok * a.ldq + (int64_t)2 * a.K * n + (int64_t)h * p + cl] : 0.f;
+        const float zz = (vc && ng == 0) ? a.z[tok * a.ldz + (int64_t)h * p + cl] : 0.f;
+        const float bt = a.beta[tok * a.H + h];
+        __syncthreads();
+        float rk = 0.f, rq = 0.f, kq = 0.f;
+#pragma unroll
+        for (int i = 0; i < MAXN; ++i) {
+            if (i < npt && n0 + i < n) {
+                const float k_ = ks[n0 + i], q_ = qs[n0 + i];
+                S[i] *= gs[n0 + i];
+                rk = fmaf(S[i], k_, rk);
+                rq = fmaf(S[i], q_, rq);
+                kq = fmaf(k_, q_, kq);
+            }
+        }
+        pk[tid] = rk;
+        pq[tid] = rq;
+        if (cl == 0) pd[ng] = kq;
+        __syncthreads();
+        rk = rq = kq = 0.f;
+        for (int j = 0; j < NG; ++j) {
+            rk += pk[j * pw + cl];
+            rq += pq[j * pw + cl];
+            kq += pd[j];
+        }
+        const float u = bt * (vv - rk);
+        const float o = vc ? fmaf(u, kq, rq) : 0.f;
+#pragma unroll
+        for (int i = 0; i < MAXN; ++i)
+            if (i < npt && n0 + i < n) S[i] = fmaf(ks[n0 + i], u, S[i]);
+        // mean square over the head's columns: a wave holds 64 of them (or all of them several times over)
+        float ss = o * o;
+        for (int m = (pw < 64 ? pw : 64) / 2; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+        if (ng == 0 && (cl & 63) == 0) red[cl >> 6] = ss;
+        __syncthreads();
+        if (ng == 0 && vc) {
+            ss = 0.f;
+            for (int j = 0; j < (pw + 63) / 64; ++j) ss += red[j];
+            const float inv = 1.0f / sqrtf(ss / (float)p + a.eps);
+            ActD<F32>::st((typename ActD<F32>::T*)a.out + tok * a.ldo + (int64_t)h * p + cl, (o * inv) * wn * sigmoid_d(zz));
+        }
+    }
+    if (vc) {
+#pragma unroll
+        for (int i = 0; i < MAXN; ++i)
+            if (i < npt && n0 + i < n) sp[(int64_t)i * p] = S[i];
+    }
+}
+
+// ---- the same recurrence in chunks of 64 tokens, for long rows -------------------------------------------------
+// Within a chunk that starts from state S0, G_t = g_1 * ... * g_t per state row (t counted within the chunk):
+//   A[t][s] = sum_i k_t[i] k_s[i] (G_t / G_s)[i]  (s < t),   B[t][s] = the same with q_t  (s <= t)
+//   (I + diag(beta) A) U = diag(beta) (V - (G * K) S0)        row by row: U = Uv - Wk S0
+//   O = (G * Q) S0 + B U,      S_end = diag(G_end) S0 + sum_s ((G_end / G_s) * k_s) u_s^T
+//   intra   per (chunk, head): A and B, the unit triangular system solved for Uv and Wk, and the operands G * Q,
+//           (G_end / G) * K (transposed) and G_end
+//   carry   per (row, head, 16 columns): U and the state from chunk to chunk
+//   inter   per (chunk, head): O, its unit-RMS, weight and sigmoid gate
+// The quotients are never formed.  A chunk is cut into four blocks of 16 tokens; G_t / G_s is the product of the gates
+// from the start of t's block to t, of whole blocks in between, and from s to the end of s's block - products of
+// numbers in (0, 1) that underflow to zero just as the token-by-token run does, whatever the gates are.  Within a
+// block a lane walks the tokens t after its s with a running product.  Matrix products are v_mfma_f32_16x16x4_f32
+// (true fp32): operand A lane (r, g) = A[r][g], B lane (r, g) = B[g][r], result lane (r, g) = C[4 g + j][r]
+// (r = lane % 16, g = lane / 16).  The contraction index is a label: in step j of a group of 16, slot g stands for
+// index 4 g + j, so a result can be the next product's operand B where it lies and operand A is a 16-byte read.
+constexpr int kDCh = 64;
+#define MV_DMFMA(acc, a_, b_) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a_, b_, acc, 0, 0, 0)
+
+// scratch per (chunk, head): qd [64][n16], wk [64][n16], kt [n16][64], uv [64][p16], bm [64][64], s0 [n16][p16], gc [n16]
+__device__ __forceinline__ int pad16(int v) { return (v + 15) & ~15; }
+
+template <int DUMMY>
+__global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int ch = blockIdx.y, h = blockIdx.x, tid = threadIdx.x;
+    const int wv = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
+    const int n = a.n, p = a.p, N = pad16(n), P = pad16(p), SN = N + 4;
+    float* Q = lds;                      // raw q, then q * (product of the gates from the block's start)
+    float* Kp = Q + kDCh * SN;           // raw k, then the same for k
+    float* Gn = Kp + kDCh * SN;          // gates, then k * (product of the gates behind the token, in its block)
+    float* Am = Gn + kDCh * SN;          // -beta A [64][68]
+    float* Di = Am + kDCh * 68;          // [4][16][20] inverses of the diagonal blocks of I + beta A
+    float* E = Di + 4 * 16 * 20;         // [4][N] products over whole blocks
+    float* bs = E + 4 * N;               // [64]
+    const int start = a.ch_start[ch], len = a.ch_len[ch], kh = h / (a.H / a.K);
+    const int64_t unit = (int64_t)ch * a.H + h;
+    const float neg_a = -expf(a.a_log[h]);
+    for (int i = tid; i < kDCh * N; i += 256) {
+        const int t = i / N, c = i - t * N;
+        float q_ = 0.f, k_ = 0.f, g_ = 1.f;
+        if (t < len && c < n) {
+            const float* qp = a.qkv + (int64_t)(start + t) * a.ldq + (int64_t)kh * n + c;
+            q_ = qp[0];
+            k_ = qp[(int64_t)a.K * n];
+            g_ = decay_gate(a.a[(int64_t)(start + t) * a.lda + (int64_t)h * n + c], a.dt_bias[(int64_t)h * n + c], neg_a);
+        }
+        Q[t * SN + c] = q_;
+        Kp[t * SN + c] = k_;
+        Gn[t * SN + c] = g_;
+    }
+    if (tid < kDCh) bs[tid] = tid < len ? a.beta[(int64_t)(start + tid) * a.H + h] : 0.f;
+    __syncthreads();
+    // the diagonal block of the wave: lane (r, g) holds column s = r, state rows 16 m + 4 g .. + 3
+    {
+        float sa[16], sb[16];
+#pragma unroll
+        for (int t = 0; t < 16; ++t) sa[t] = sb[t] = 0.f;
+        const float* q0 = Q + 16 * wv * SN + 4 * g;
+        const float* k0 = Kp + 16 * wv * SN + 4 * g;
+        const float* g0 = Gn + 16 * wv * SN + 4 * g;
+        for (int m = 0; m < N; m += 16) {
+            const float4 ks = *reinterpret_cast<const float4*>(k0 + r * SN + m);
+            float4 w = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+            for (int t = 0; t < 16; ++t) {
+                const float4 gt = *reinterpret_cast<const float4*>(g0 + t * SN + m);
+                const float4 kt = *reinterpret_cast<const float4*>(k0 + t * SN + m);
+                const float4 qt = *reinterpret_cast<const float4*>(q0 + t * SN + m);
+                const bool self = t == r;
+                w.x = self ? ks.x : w.x * gt.x;
+                w.y = self ? ks.y : w.y * gt.y;
+                w.z = self ? ks.z : w.z * gt.z;
+                w.w = self ? ks.w : w.w * gt.w;
+                sa[t] = fmaf(kt.x, w.x, fmaf(kt.y, w.y, fmaf(kt.z, w.z, fmaf(kt.w, w.w, sa[t]))));
+                sb[t] = fmaf(qt.x, w.x, fmaf(qt.y, w.y, fmaf(qt.z, w.z, fmaf(qt.w, w.w, sb[t]))));
+            }
+        }
+        float* bm = a.bm + unit * (kDCh * kDCh);
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            float x = sa[t], y = sb[t];
+            x += __shfl_xor(x, 16, 64);
+            x += __shfl_xor(x, 32, 64);
+            y += __shfl_xor(y, 16, 64);
+            y += __shfl_xor(y, 32, 64);
+            if ((t >> 2) == g) {
+                const int tt = 16 * wv + t;
+                Am[tt * 68 + 16 * wv + r] = r < t ? -bs[tt] * x : 0.f;
+                bm[tt * kDCh + 16 * wv + r] = r <= t ? y : 0.f;
+            }
+        }
+    }
+    __syncthreads();
+    // products of the gates, in place: thread per (block, state row)
+    for (int i = tid; i < 4 * N; i += 256) {
+        const int blk = i / N, c = i - blk * N;
+        float* qc = Q + 16 * blk * SN + c;
+        float* kc = Kp + 16 * blk * SN + c;
+        float* gc = Gn + 16 * blk * SN + c;
+        float gt[16], kk[16];
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            gt[t] = gc[t * SN];
+            kk[t] = kc[t * SN];
+        }
+        float suf = 1.f;
+#pragma unroll
+        for (int t = 15; t >= 0; --t) {
+            gc[t * SN] = kk[t] * suf;
+            suf *= gt[t];
+        }
+        float pre = 1.f;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            pre *= gt[t];
+            kc[t * SN] = kk[t] * pre;
+            qc[t * SN] *= pre;
+        }
+        E[blk * N + c] = pre;
+    }
+    // inverse of the wave's unit triangular diagonal block: lane r owns column r, forward substitution
+    if (g == 0) {
+        float x[16];
+        const float* m = Am + (16 * wv) * 68 + 16 * wv;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            float s = t == r ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < t; ++j) s = fmaf(m[t * 68 + j], x[j], s);
+            x[t] = s;
+            Di[(wv * 16 + t) * 20 + r] = s;
+        }
+    }
+    __syncthreads();
+    // blocks below the diagonal: six block pairs, A and B each, three products a wave
+    for (int x = 0; x < 3; ++x) {
+        const int id = wv * 3 + x, pair = id >> 1;
+        const bool isb = id & 1;
+        const int I = pair == 0 ? 1 : (pair < 3 ? 2 : 3), J = pair == 0 ? 0 : (pair < 3 ? pair - 1 : pair - 3);
+        f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        const float* ar = (isb ? Q : Kp) + (16 * I + r) * SN + 4 * g;
+        const float* br = Gn + (16 * J + r) * SN + 4 * g;
+        for (int m = 0; m < N; m += 16) {
+            const float4 av = *reinterpret_cast<const float4*>(ar + m);
+            float4 bv = *reinterpret_cast<const float4*>(br + m);
+            for (int M = J + 1; M < I; ++M) {
+                const float4 e = *reinterpret_cast<const float4*>(E + M * N + m + 4 * g);
+                bv.x *= e.x;
+                bv.y *= e.y;
+                bv.z *= e.z;
+                bv.w *= e.w;
+            }
+            MV_DMFMA(acc, av.x, bv.x);
+            MV_DMFMA(acc, av.y, bv.y);
+            MV_DMFMA(acc, av.z, bv.z);
+            MV_DMFMA(acc, av.w, bv.w);
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int t = 16 * I + 4 * g + j, s = 16 * J + r;
+            if (isb) a.bm[unit * (kDCh * kDCh) + t * kDCh + s] = acc[j];
+            else Am[t * 68 + s] = -bs[t] * acc[j];
+        }
+    }
+    // operands of the other two kernels
+    float* qd = a.qd + unit * (kDCh * N);
+    for (int i = tid; i < kDCh * N; i += 256) {
+        const int t = i / N, c = i - t * N;
+        float v = Q[t * SN + c];
+        for (int M = 0; M < (t >> 4); ++M) v *= E[M * N + c];
+        qd[i] = v;
+    }
+    float* kt = a.kt + unit * (kDCh * N);
+    for (int i = tid; i < kDCh * N; i += 256) {
+        const int c = i >> 6, s = i & 63;
+        float v = Gn[s * SN + c];
+        for (int M = (s >> 4) + 1; M < 4; ++M) v *= E[M * N + c];
+        kt[i] = v;
+    }
+    for (int c = tid; c < N; c += 256) a.gc[unit * N + c] = ((E[c] * E[N + c]) * E[2 * N + c]) * E[3 * N + c];
+    __syncthreads();
+    // the triangular system, 16 columns at a time: first those of V, then those of G * K
+    const int pt = P / 16, ntile = pt + N / 16;
+    float* uv = a.uv + unit * (kDCh * P);
+    float* wk = a.wk + unit * (kDCh * N);
+    for (int tile = wv; tile < ntile; tile += 4) {
+        const bool isv = tile < pt;
+        const int c = 16 * (isv ? tile : tile - pt) + r;
+        f32x4_t X[4];
+        float e = 1.f;           // product of the blocks before I for column c of G * K
+#pragma unroll
+        for (int I = 0; I < 4; ++I) {
+            f32x4_t acc;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int t = 16 * I + 4 * g + j;
+                float v;
+                if (isv) v = (t < len && c < p) ? a.qkv[(int64_t)(start + t) * a.ldq + (int64_t)2 * a.K * n + (int64_t)h * p + c] : 0.f;
+                else v = Kp[t * SN + c] * e;
+                acc[j] = bs[t] * v;
+            }
+            if (!isv) e *= E[I * N + c];
+#pragma unroll
+            for (int J = 0; J < I; ++J) {
+                const float4 m = *reinterpret_cast<const float4*>(Am + (16 * I + r) * 68 + 16 * J + 4 * g);
+                MV_DMFMA(acc, m.x, X[J][0]);
+                MV_DMFMA(acc, m.y, X[J][1]);
+                MV_DMFMA(acc, m.z, X[J][2]);
+                MV_DMFMA(acc, m.w, X[J][3]);
+            }
+            const float4 d = *reinterpret_cast<const float4*>(Di + (16 * I + r) * 20 + 4 * g);
+            X[I] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            MV_DMFMA(X[I], d.x, acc[0]);
+            MV_DMFMA(X[I], d.y, acc[1]);
+            MV_DMFMA(X[I], d.z, acc[2]);
+            MV_DMFMA(X[I], d.w, acc[3]);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int t = 16 * I + 4 * g + j;
+                if (isv) uv[t * P + c] = X[I][j];
+                else wk[t * N + c] = X[I][j];
+            }
+        }
+    }
+}
+
+// One workgroup per (head, 16 state columns, row).  Wave w forms U for the tokens 16 w .. + 15 of a chunk and owns the
+// state rows of the 16-row tiles w, w + 4, ...; the state (as operand) and U pass through LDS.  NT: 16-row tiles.
+template <int NT>
+__global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
+    constexpr int OWN = (NT + 3) / 4;
+    __shared__ float Ss[NT * 16][20];
+    __shared__ float Us[kDCh][20];
+    const int h = blockIdx.x, c0 = blockIdx.y * 16, b = blockIdx.z;
+    const int nch = a.row_nch[b];
+    if (nch == 0) return;
+    const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
+    const int n = a.n, p = a.p, N = pad16(n), P = pad16(p), nt = N / 16;
+    const bool carried = a.r.row_ctx[b] > 0;
+    float* st = a.state + ((int64_t)a.r.row_slot[b] * a.H + h) * n * p + c0 + r;
+    const bool vc = c0 + r < p;
+    f32x4_t S[OWN];
+#pragma unroll
+    for (int o = 0; o < OWN; ++o) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int i = 16 * (wv + 4 * o) + 4 * g + j;
+            S[o][j] = (carried && vc && i < n) ? st[(int64_t)i * p] : 0.f;
+            if (i < NT * 16) Ss[i][r] = S[o][j];
+        }
+    }
+    const int64_t u0 = (int64_t)a.row_ch0[b] * a.H + h;
+    float4 wk[NT], kt[OWN][4], gm[OWN];
+    f32x4_t uv;
+    auto fetch = [&](int64_t unit) {
+        const float* w = a.wk + unit * (kDCh * N) + (16 * wv + r) * N + 4 * g;
+#pragma unroll
+        for (int i = 0; i < NT; ++i)
+            if (i < nt) wk[i] = *reinterpret_cast<const float4*>(w + 16 * i);
+#pragma unroll
+        for (int o = 0; o < OWN; ++o) {
+            const int it = wv + 4 * o;
+            if (it < nt) {
+                const float* k = a.kt + unit * (kDCh * N) + (16 * it + r) * kDCh + 4 * g;
+#pragma unroll
+                for (int t = 0; t < 4; ++t) kt[o][t] = *reinterpret_cast<const float4*>(k + 16 * t);
+                gm[o] = *reinterpret_cast<const float4*>(a.gc + unit * N + 16 * it + 4 * g);
+            }
+        }
+        const float* up = a.uv + unit * (kDCh * P) + (16 * wv + 4 * g) * P + c0 + r;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) uv[j] = up[j * P];
+    };
+    fetch(u0);
+    __syncthreads();
+    for (int c = 0; c < nch; ++c) {
+        const int64_t unit = u0 + (int64_t)c * a.H;
+        // two accumulators: neighbouring products do not wait for each other
+        f32x4_t x0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, x1 = x0;
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+            if (i < nt) {
+                const int k = 16 * i + 4 * g;
+                MV_DMFMA(x0, wk[i].x, Ss[k][r]);
+                MV_DMFMA(x1, wk[i].y, Ss[k + 1][r]);
+                MV_DMFMA(x0, wk[i].z, Ss[k + 2][r]);
+                MV_DMFMA(x1, wk[i].w, Ss[k + 3][r]);
+            }
+        }
+        float* up = a.uv + unit * (kDCh * P) + (16 * wv + 4 * g) * P + c0 + r;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const float u = uv[j] - (x0[j] + x1[j]);
+            Us[16 * wv + 4 * g + j][r] = u;
+            up[j * P] = u;
+        }
+        float* sp = a.s0 + unit * ((int64_t)N * P) + c0 + r;
+#pragma unroll
+        for (int o = 0; o < OWN; ++o) {
+            const int it = wv + 4 * o;
+            if (it < nt) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) sp[(int64_t)(16 * it + 4 * g + j) * P] = S[o][j];    // what this chunk starts from
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int o = 0; o < OWN; ++o) {
+            const int it = wv + 4 * o;
+            if (it >= nt) continue;
+            f32x4_t y0 = f32x4_t{S[o][0] * gm[o].x, S[o][1] * gm[o].y, S[o][2] * gm[o].z, S[o][3] * gm[o].w};
+            f32x4_t y1 = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                const int k = 16 * t + 4 * g;
+                MV_DMFMA(y0, kt[o][t].x, Us[k][r]);
+                MV_DMFMA(y1, kt[o][t].y, Us[k + 1][r]);
+                MV_DMFMA(y0, kt[o][t].z, Us[k + 2][r]);
+                MV_DMFMA(y1, kt[o][t].w, Us[k + 3][r]);
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                S[o][j] = y0[j] + y1[j];
+                Ss[16 * it + 4 * g + j][r] = S[o][j];
+            }
+        }
+        if (c + 1 < nch) fetch(unit + a.H);
+        __syncthreads();
+    }
+#pragma unroll
+    for (int o = 0; o < OWN; ++o)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int i = 16 * (wv + 4 * o) + 4 * g + j;
+            if (vc && i < n) st[(int64_t)i * p] = S[o][j];
+        }
+}
+
+// One workgroup per (head, chunk), 16 tokens a wave: lane (r, g) ends with token r, columns 16 ct + 4 g .. + 3.
+template <bool F32, int PT>
+__global__ __launch_bounds__(256) void delta_chunk_inter_kernel(DeltaArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int h = blockIdx.x, ch = blockIdx.y, tid = threadIdx.x;
+    const int wv = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
+    const int p = a.p, N = pad16(a.n), P = pad16(p), pt = P / 16, SP = P + 4;
+    const int64_t unit = (int64_t)ch * a.H + h;
+    const int start = a.ch_start[ch], len = a.ch_len[ch];
+    f32x4_t o[PT];
+#pragma unroll
+    for (int ct = 0; ct < PT; ++ct) o[ct] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const float* qd = a.qd + unit * (kDCh * N) + (16 * wv + r) * N + 4 * g;
+    const float* bm = a.bm + unit * (kDCh * kDCh) + (16 * wv + r) * kDCh + 4 * g;
+    const float* s0 = a.s0 + unit * ((int64_t)N * P);
+    const float* uv = a.uv + unit * (kDCh * P);
+    const int P4 = P / 4;
+    // 64 rows of the right-hand operand at a time: the state's, then U's
+    for (int k0 = 0; k0 < N + kDCh; k0 += kDCh) {
+        const bool isu = k0 >= N;
+        const int rows = isu ? kDCh : (N - k0 < kDCh ? N - k0 : kDCh);
+        const float* src = isu ? uv : s0 + (int64_t)k0 * P;
+        __syncthreads();
+        for (int i = tid; i < rows * P4; i += 256) {
+            const int rr = i / P4, cc = i - rr * P4;
+            *reinterpret_cast<float4*>(lds + rr * SP + 4 * cc) = *reinterpret_cast<const float4*>(src + (int64_t)rr * P + 4 * cc);
+        }
+        __syncthreads();
+        const int top = isu ? 16 * (wv + 1) : rows;      // tokens behind the wave's own do not enter
+        for (int k = 0; k < top; k += 16) {
+            const float4 w = *reinterpret_cast<const float4*>(isu ? bm + k : qd + k0 + k);
+            const float* s = lds + (k + 4 * g) * SP + r;
+#pragma unroll
+            for (int ct = 0; ct < PT; ++ct) {
+                if (ct < pt) {
+                    MV_DMFMA(o[ct], s[16 * ct], w.x);
+                    MV_DMFMA(o[ct], s[SP + 16 * ct], w.y);
+                    MV_DMFMA(o[ct], s[2 * SP + 16 * ct], w.z);
+                    MV_DMFMA(o[ct], s[3 * SP + 16 * ct], w.w);
+                }
+            }
+        }
+        if (isu) break;
+        if (k0 + kDCh >= N) k0 = N - kDCh;               // U's rows come next, whatever N is
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int ct = 0; ct < PT; ++ct)
+        if (ct < pt) ss += o[ct][0] * o[ct][0] + o[ct][1] * o[ct][1] + o[ct][2] * o[ct][2] + o[ct][3] * o[ct][3];
+    ss += __shfl_xor(ss, 16, 64);
+    ss += __shfl_xor(ss, 32, 64);
+    const int t = 16 * wv + r;
+    if (t >= len) return;
+    const float inv = 1.0f / sqrtf(ss / (float)p + a.eps);
+    const float* zp = a.z + (int64_t)(start + t) * a.ldz + (int64_t)h * p;
+    typename ActD<F32>::T* op = (typename ActD<F32>::T*)a.out + (int64_t)(start + t) * a.ldo + (int64_t)h * p;
+#pragma unroll
+    for (int ct = 0; ct < PT; ++ct) {
+        if (ct >= pt) continue;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int c = 16 * ct + 4 * g + j;
+            if (c < p) ActD<F32>::st(op + c, (o[ct][j] * inv) * a.norm[c] * sigmoid_d(zp[c]));
+        }
+    }
+}
+
+static size_t delta_intra_lds(int n) {
+    const int N = (n + 15) & ~15;
+    return ((size_t)3 * kDCh * (N + 4) + kDCh * 68 + 4 * 16 * 20 + 4 * N + kDCh) * sizeof(float);
+}
+
+}  // namespace mv
+
+extern "C" {
+
+int mv_delta_prep(const float* proj, int64_t ldp, int b_off, int low_off, int low_n, float* state, const float* wt,
+                  float* out, int64_t ldo, float* beta, void* low, int64_t ldl, const int32_t* tok_row,
+                  const int32_t* row_start, const int32_t* row_len, const int32_t* row_ctx, const int32_t* row_slot,
+                  int tokens, int rows, int kv_heads, int n, int heads, int p, int taps, float eps, float q_scale,
+                  int f32, mv_stream_t stream) {
+    using namespace mv;
+    if (tokens < 0 || rows < 0 || kv_heads <= 0 || heads <= 0 || heads % kv_heads || n <= 0 || p <= 0 || taps < 1 ||
+        taps > kDeltaMaxTaps || low_n < 0)
+        return MV_ERR_INVALID_ARG;
+    if (n > kDeltaMaxN) return MV_ERR_UNSUPPORTED;
+    if (tokens == 0) return MV_OK;
+    const int C = 2 * kv_heads * n + heads * p;
+    if (!proj || (taps > 1 && !state) || !wt || !out || !beta || (low_n > 0 && !low) || !tok_row || !row_start ||
+        !row_len || !row_ctx || !row_slot || ldp < C || ldo < C || b_off < C || ldp < b_off + heads ||
+        (low_n > 0 && (low_off < C || ldp < low_off + low_n || ldl < low_n)))
+        return MV_ERR_INVALID_ARG;
+    DeltaPrepArgs a;
+    a.proj = proj; a.ldp = ldp; a.ldo = ldo; a.ldl = ldl; a.b_off = b_off; a.low_off = low_off; a.low_n = low_n;
+    a.state = state; a.wt = wt; a.out = out; a.beta = beta; a.low = low;
+    a.r = DeltaRows{tok_row, row_start, row_len, row_ctx, row_slot};
+    a.T = tokens; a.K = kv_heads; a.n = n; a.H = heads; a.p = p; a.taps = taps;
+    a.in_place = tokens == rows && taps > 1;       // every row has one token
+    a.eps = eps; a.qscale = q_scale;
+    hipStream_t s = (hipStream_t)stream;
+    const int units = 2 * kv_heads + (heads * p + 255) / 256 + 1;
+    if (units > 65535) return MV_ERR_UNSUPPORTED;
+    const dim3 grid((tokens + 3) / 4, units);
+    if (f32) hipLaunchKernelGGL(delta_prep_kernel<true>, grid, dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(delta_prep_kernel<false>, grid, dim3(256), 0, s, a);
+    if (taps > 1 && !a.in_place) {
+        const int64_t work = (int64_t)rows * C;
+        hipLaunchKernelGGL(delta_conv_state_kernel, dim3((unsigned)((work + 255) / 256)), dim3(256), 0, s, a, rows);
+    }
+    return check_launch();
+}
+
+int mv_delta_chunked_ok(int n, int p) {
+    return n > 0 && p > 0 && n <= 160 && p <= 256 && mv::delta_intra_lds(n) <= 158 * 1024;
+}
+
+int64_t mv_delta_scratch_floats(int n, int p) {
+    const int64_t N = (n + 15) & ~15, P = (p + 15) & ~15;
+    return 3 * mv::kDCh * N + mv::kDCh * P + mv::kDCh * mv::kDCh + N * P + N;
+}
+
+int mv_delta_rule(const float* qkv, int64_t ldq, const float* gate_in, int64_t lda, const float* z, int64_t ldz,
+                  const float* beta, const float* dt_bias, const float* a_log, const float* norm, float* state,
+                  void* out, int64_t ldo, const int32_t* row_start, const int32_t* row_len, const int32_t* row_ctx,
+                  const int32_t* row_slot, int rows, int kv_heads, int heads, int n, int p, float eps, float* scratch,
+                  const int32_t* ch_start, const int32_t* ch_len, const int32_t* row_ch0, const int32_t* row_nch,
+                  int chunks, int max_len, int short_tokens, int f32, mv_stream_t stream) {
+    using namespace mv;
+    if (rows < 0 || kv_heads <= 0 || heads <= 0 || heads % kv_heads || n <= 0 || p <= 0 || chunks < 0)
+        return MV_ERR_INVALID_ARG;
+    if (p > 256 || n > kDeltaMaxN || rows > 65535 || chunks > 65535) return MV_ERR_UNSUPPORTED;
+    if (rows == 0) return MV_OK;
+    const int64_t cq = 2 * (int64_t)kv_heads * n + (int64_t)heads * p;
+    if (!qkv || !gate_in || !z || !beta || !dt_bias || !a_log || !norm || !state || !out || !row_start || !row_len ||
+        !row_ctx || !row_slot || ldq < cq || lda < (int64_t)heads * n || ldz < (int64_t)heads * p ||
+        ldo < (int64_t)heads * p)
+        return MV_ERR_INVALID_ARG;
+    if (chunks > 0 && (!scratch || !ch_start || !ch_len || !row_ch0 || !row_nch || max_len <= 0 || !aligned16(scratch)))
+        return MV_ERR_INVALID_ARG;
+    if (chunks > 0 && !mv_delta_chunked_ok(n, p)) return MV_ERR_UNSUPPORTED;
+    DeltaArgs a;
+    a.qkv = qkv; a.a = gate_in; a.z = z; a.beta = beta; a.dt_bias = dt_bias; a.a_log = a_log; a.norm = norm;
+    a.ldq = ldq; a.lda = lda; a.ldz = ldz; a.ldo = ldo; a.state = state; a.out = out;
+    a.r = DeltaRows{nullptr, row_start, row_len, row_ctx, row_slot};
+    a.K = kv_heads; a.H = heads; a.n = n; a.p = p; a.max_len = chunks > 0 ? max_len : 0; a.eps = eps;
+    a.ch_start = ch_start; a.ch_len = ch_len; a.row_ch0 = row_ch0; a.row_nch = row_nch;
+    hipStream_t s = (hipStream_t)stream;
+    if (chunks == 0 || short_tokens != 0) {
+        int pw = 16;
+        while (pw < p) pw *= 2;
+        int nt = 256;
+        while (nt < 1024 && (int64_t)n * pw > (int64_t)nt * 16) nt *= 2;
+        const int ng = nt / pw, npt = (n + ng - 1) / ng;
+        const size_t lds = ((size_t)3 * n + 2 * nt + ng + 8) * sizeof(float);
+        const dim3 grid(heads, rows);
+#define MV_DELTA_SCAN(M_)                                                                                       \
+    do {                                                                                                       \
+        if (f32) hipLaunchKernelGGL((delta_scan_kernel<true, M_>), grid, dim3(nt), lds, s, a, pw);               \
+        else hipLaunchKernelGGL((delta_scan_kernel<false, M_>), grid, dim3(nt), lds, s, a, pw);                  \
+    } while (0)
+        if (npt <= 4) MV_DELTA_SCAN(4);
+        else if (npt <= 8) MV_DELTA_SCAN(8);
+        else if (npt <= 16) MV_DELTA_SCAN(16);
+        else if (npt <= 32) MV_DELTA_SCAN(32);
+        else if (npt <= 64) MV_DELTA_SCAN(64);
+        else return MV_ERR_UNSUPPORTED;
+#undef MV_DELTA_SCAN
+    }
+    if (chunks > 0) {
+        const int64_t N = (n + 15) & ~15, P = (p + 15) & ~15, U = (int64_t)chunks * heads;
+        a.qd = scratch;
+        a.wk = a.qd + U * kDCh * N;
+        a.kt = a.wk + U * kDCh * N;
+        a.uv = a.kt + U * kDCh * N;
+        a.bm = a.uv + U * kDCh * P;
+        a.s0 = a.bm + U * kDCh * kDCh;
+        a.gc = a.s0 + U * N * P;
+        const size_t lds1 = delta_intra_lds(n), lds2 = (size_t)kDCh * (P + 4) * sizeof(float);
+        static LdsOptIn o1, o2[2][4];
+        if (int rc = ensure_dynamic_lds((const void*)delta_chunk_intra_kernel<0>, lds1, o1)) return rc;
+        hipLaunchKernelGGL(delta_chunk_intra_kernel<0>, dim3(heads, chunks), dim3(256), lds1, s, a);
+        const dim3 gc(heads, (unsigned)(P / 16), rows);
+        if (N <= 32) hipLaunchKernelGGL(delta_chunk_carry_kernel<2>, gc, dim3(256), 0, s, a);
+        else if (N <= 64) hipLaunchKernelGGL(delta_chunk_carry_kernel<4>, gc, dim3(256), 0, s, a);
+        else if (N <= 128) hipLaunchKernelGGL(delta_chunk_carry_kernel<8>, gc, dim3(256), 0, s, a);
+        else hipLaunchKernelGGL(delta_chunk_carry_kernel<10>, gc, dim3(256), 0, s, a);
+        const dim3 gi(heads, chunks);
+#define MV_DELTA_INTER(F32_, PT_, IDX_)                                                                                    \
+    do {                                                                                                               \
+        if (int rc = ensure_dynamic_lds((const void*)delta_chunk_inter_kernel<F32_, PT_>, lds2, o2[F32_][IDX_])) return rc;  \
+        hipLaunchKernelGGL((delta_chunk_inter_kernel<F32_, PT_>), gi, dim3(256), lds2, s, a);                             \
+    } while (0)
+        if (f32) {
+            if (P <= 32) MV_DELTA_INTER(true, 2, 0); else if (P <= 64) MV_DELTA_INTER(true, 4, 1);
+            else if (P <= 128) MV_DELTA_INTER(true, 8, 2); else MV_DELTA_INTER(true, 16, 3);
+        } else {
+            if (P <= 32) MV_DELTA_INTER(false, 2, 0); else if (P <= 64) MV_DELTA_INTER(false, 4, 1);
+            else if (P <= 128) MV_DELTA_INTER(false, 8, 2); else MV_DELTA_INTER(false, 16, 3);
+        }
+#undef MV_DELTA_INTER
+    }
+    return check_launch();
+}
+
+}  // extern "C"

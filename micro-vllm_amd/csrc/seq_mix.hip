@@ -23,7 +23,11 @@
 //                                  key as projected into the value page (attention whose values are its keys)
 //   window_attn                    softmax attention over the last `window` positions (and, where asked for, the
 //                                  sequence's first `keep_first` positions) with a per-head linear distance
-//                                  penalty and / or a per-head sink in the denominator
+//                                  penalty and / or a per-head sink in the denominator; optionally a sigmoid gate
+//                                  on every output value
+//   qkv_norm_rotary_store          biases on q, k and v, RMS norms over ALL heads of q and of k at once, rotation of
+//                                  both, values mixed with another layer's for the same token; keys and values into
+//                                  their pages
 // All of it in fp32; the activation type (bf16 or fp32) only concerns what goes to a projection or
 // into the key/value pages.
 #include "common.h"
@@ -43,6 +47,7 @@ template <> struct ActS<false> {
 };
 
 __device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
+__device__ __forceinline__ float sigmoid_f(float v) { return 1.0f / (1.0f + expf(-v)); }
 
 struct StepRows {
     const int* tok_row;    // [T] row of each token
@@ -548,8 +553,8 @@ __global__ __launch_bounds__(256) void rotary_pairs_kernel(float* x, int64_t ld,
 template <bool F32>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* y, int64_t ldy, const float* gate,
                                                                int64_t ldg, const float* w, void* out_, int64_t ldo,
-                                                               int rows, int n, int groups, int gate_first,
-                                                               float eps) {
+                                                               int rows, int n, int groups, int mode,
+                                                               int w_shared, float eps) {
     typedef typename ActS<F32>::T T;
     T* out = (T*)out_;
     const int unit = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
@@ -559,14 +564,14 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* y, i
     const float* gr = gate + (int64_t)row * ldg + (int64_t)g * gs;
     float ss = 0.f;
     for (int c = lane; c < gs; c += 64) {
-        const float u = gate_first ? yr[c] * silu_f(gr[c]) : yr[c];
+        const float u = mode == 1 ? yr[c] * silu_f(gr[c]) : yr[c];
         ss += u * u;
     }
     ss = wave_sum(ss);
     const float inv = 1.0f / sqrtf(ss / (float)gs + eps);
     for (int c = lane; c < gs; c += 64) {
-        float u = gate_first ? (yr[c] * silu_f(gr[c])) * inv : (yr[c] * inv) * silu_f(gr[c]);
-        if (w) u *= w[g * gs + c];
+        float u = mode == 1 ? (yr[c] * silu_f(gr[c])) * inv : (yr[c] * inv) * (mode == 2 ? sigmoid_f(gr[c]) : silu_f(gr[c]));
+        if (w) u *= w[w_shared ? c : g * gs + c];
         ActS<F32>::st(out + (int64_t)row * ldo + (int64_t)g * gs + c, u);
     }
 }
@@ -688,6 +693,101 @@ __global__ __launch_bounds__(256) void qk_rotary_store_kernel(float* qk, int64_t
     }
 }
 
+// One workgroup per token.  qkv row: q [H * d] | k [G * d] | v [G * dv], as one projection leaves them.  Each of q and k gets
+// its bias and an RMS norm over the WHOLE of it (plain weights; NULL: no norm), then the rotation of its heads' first
+// `rot` dimensions (adjacent pairs or halves; the angle is formed in fp64, once per token for all heads); q stays in
+// place, k goes to the key page.  v gets its bias; mix 1: v is kept in vfirst [T, G * dv]; mix 2: v = (1 - lam) v + lam
+// vfirst; v goes to the value page.
+template <bool F32>
+__global__ __launch_bounds__(256) void qkv_norm_rotary_store_kernel(float* qkv, int64_t ld, const float* qb,
+                                                                    const float* kb, const float* vb, const float* qn,
+                                                                    const float* kn, float eps, const double* inv_freq,
+                                                                    float* vfirst, int mix, float lam, void* kc_,
+                                                                    void* vc_, PagedRows pr, int H, int G, int d,
+                                                                    int dv, int rot, int adjacent) {
+    typedef typename ActS<F32>::T T_;
+    extern __shared__ float ang[];     // [rot / 2] cosines, then sines
+    __shared__ float red[8];
+    T_* kc = (T_*)kc_;
+    T_* vc = (T_*)vc_;
+    const int t = blockIdx.x, tid = threadIdx.x, pos = pr.tok_pos[t];
+    float* q = qkv + (int64_t)t * ld;
+    float* k = q + (int64_t)H * d;
+    const float* v = k + (int64_t)G * d;
+    const int pg = pr.block_table[(int64_t)pr.tok_row[t] * pr.bt_stride + pos / pr.page];
+    const int64_t slot = (int64_t)pg * pr.page + pos % pr.page;
+    const int half = rot / 2;
+    for (int i = tid; i < half; i += 256) {
+        const double a = (double)pos * inv_freq[i];
+        ang[i] = (float)cos(a);
+        ang[half + i] = (float)sin(a);
+    }
+    float sq = 0.f, sk = 0.f;
+    if (qn) {
+#pragma unroll 4
+        for (int c = tid; c < H * d; c += 256) {
+            const float x = qb ? q[c] + qb[c] : q[c];
+            sq += x * x;
+        }
+    }
+    if (kn) {
+#pragma unroll 4
+        for (int c = tid; c < G * d; c += 256) {
+            const float x = kb ? k[c] + kb[c] : k[c];
+            sk += x * x;
+        }
+    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((tid & 63) == 0) {
+        red[tid >> 6] = sq;
+        red[4 + (tid >> 6)] = sk;
+    }
+    __syncthreads();
+    const float iq = qn ? 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)(H * d) + eps) : 1.f;
+    const float ik = kn ? 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)(G * d) + eps) : 1.f;
+    const int per = d - half;         // a head's items: `half` rotated pairs, then the dimensions behind them
+    for (int i = tid; i < (H + G) * per; i += 256) {
+        const int u = i / per, j = i - u * per;
+        const bool isq = u < H;
+        const int base = isq ? u * d : (u - H) * d;
+        float* src = isq ? q : k;
+        const float* b = isq ? qb : kb;
+        const float* w = isq ? qn : kn;
+        const float inv = isq ? iq : ik;
+        if (j < half) {
+            const int a0 = base + (adjacent ? 2 * j : j), a1 = base + (adjacent ? 2 * j + 1 : j + half);
+            float x0 = b ? src[a0] + b[a0] : src[a0], x1 = b ? src[a1] + b[a1] : src[a1];
+            if (w) {
+                x0 = (x0 * inv) * w[a0];
+                x1 = (x1 * inv) * w[a1];
+            }
+            const float cs = ang[j], sn = ang[half + j];
+            const float r0 = x0 * cs - x1 * sn, r1 = x1 * cs + x0 * sn;
+            if (isq) {
+                q[a0] = r0;
+                q[a1] = r1;
+            } else if (pg >= 0) {
+                ActS<F32>::st(kc + slot * G * d + a0, r0);
+                ActS<F32>::st(kc + slot * G * d + a1, r1);
+            }
+        } else {
+            const int c = base + half + j;
+            float x = b ? src[c] + b[c] : src[c];
+            if (w) x = (x * inv) * w[c];
+            if (isq) q[c] = x;
+            else if (pg >= 0) ActS<F32>::st(kc + slot * G * d + c, x);
+        }
+    }
+    for (int c = tid; c < G * dv; c += 256) {
+        float x = vb ? v[c] + vb[c] : v[c];
+        float* f = mix ? vfirst + (int64_t)t * G * dv + c : nullptr;
+        if (mix == 1) *f = x;
+        else if (mix == 2) x = (1.0f - lam) * x + lam * *f;
+        if (pg >= 0) ActS<F32>::st(vc + slot * G * dv + c, x);
+    }
+}
+
 // value of channel c at token t under a causal convolution of `taps` taps whose first inputs come from the slot
 __device__ __forceinline__ float conv_at(const float* in, int64_t ldi, const float* state, const float* w,
                                          const StepRows& r, int t, int c, int C, int taps) {
@@ -760,7 +860,8 @@ __global__ __launch_bounds__(64 * NW) void window_attn_kernel(const float* q, in
                                                           const void* vc_, void* out_, int64_t ldo, PagedRows pr,
                                                           const float* slopes, int T, int H, int G, int d, int dv,
                                                           float scale, int window, const int* row_len, int max_len,
-                                                          int keep_first, const float* sinks) {
+                                                          int keep_first, const float* sinks, const float* gate,
+                                                          int64_t ldg) {
     typedef typename ActS<F32>::T T_;
     extern __shared__ float lds[];
     if (max_len > 0 && row_len[pr.tok_row[blockIdx.x / H]] > max_len) return;   // the tiled kernel's rows
@@ -879,7 +980,9 @@ __global__ __launch_bounds__(64 * NW) void window_attn_kernel(const float* q, in
                 float o = 0.f;
 #pragma unroll
                 for (int w = 0; w < NW; ++w) o = fmaf(aa[w * dv + c], w4[w], o);
-                ActS<F32>::st(out + (int64_t)t * ldo + (int64_t)h * dv + c, o / L);
+                o /= L;
+                if (gate) o *= sigmoid_f(gate[(int64_t)t * ldg + (int64_t)h * dv + c]);
+                ActS<F32>::st(out + (int64_t)t * ldo + (int64_t)h * dv + c, o);
             }
         }
     }
@@ -902,7 +1005,7 @@ __global__ __launch_bounds__(256) void window_attn_group_kernel(const float* q, 
                                                                 PagedRows pr, const float* slopes, const float* sinks,
                                                                 int H, int G, int d, int dv, float scale, int window,
                                                                 int keep_first, const int* row_len, int max_len,
-                                                                int splits, int vec) {
+                                                                int splits, int vec, const float* gate, int64_t ldg) {
     typedef typename ActS<F32>::T T_;
     constexpr int VEC = F32 ? 4 : 8;
     extern __shared__ float lds[];
@@ -1112,7 +1215,9 @@ __global__ __launch_bounds__(256) void window_attn_group_kernel(const float* q, 
                 L = L * f + expf(sk - mf);
                 o *= f;
             }
-            ActS<F32>::st((T_*)out_ + (int64_t)t * ldo + (int64_t)h * dv + c, o / L);
+            o /= L;
+            if (gate) o *= sigmoid_f(gate[(int64_t)t * ldg + (int64_t)h * dv + c]);
+            ActS<F32>::st((T_*)out_ + (int64_t)t * ldo + (int64_t)h * dv + c, o);
         } else {
             float* dst = part + (((int64_t)t * H + h) * splits + split) * (dv + 2);
             if (c == 0) {
@@ -1128,7 +1233,8 @@ __global__ __launch_bounds__(256) void window_attn_group_kernel(const float* q, 
 template <bool F32>
 __global__ __launch_bounds__(64) void window_attn_merge_kernel(const float* part, void* out_, int64_t ldo,
                                                                const int* tok_row, const float* sinks, int H, int dv,
-                                                               int splits, const int* row_len, int max_len) {
+                                                               int splits, const int* row_len, int max_len,
+                                                               const float* gate, int64_t ldg) {
     typedef typename ActS<F32>::T T_;
     const int t = blockIdx.x / H, h = blockIdx.x % H, lane = threadIdx.x;
     if (max_len > 0 && row_len[tok_row[t]] > max_len) return;
@@ -1146,7 +1252,9 @@ __global__ __launch_bounds__(64) void window_attn_merge_kernel(const float* part
             const float ms = src[(int64_t)s2 * (dv + 2)];
             if (ms != -INFINITY) o = fmaf(src[(int64_t)s2 * (dv + 2) + 2 + c], expf(ms - M), o);
         }
-        ActS<F32>::st((T_*)out_ + (int64_t)t * ldo + (int64_t)h * dv + c, o / L);
+        o /= L;
+        if (gate) o *= sigmoid_f(gate[(int64_t)t * ldg + (int64_t)h * dv + c]);
+        ActS<F32>::st((T_*)out_ + (int64_t)t * ldo + (int64_t)h * dv + c, o);
     }
 }
 
@@ -1163,7 +1271,8 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
                                                                const uint16_t* vc, uint16_t* out, int64_t ldo,
                                                                PagedRows pr, const int* ch_start, const int* ch_len,
                                                                const float* slopes, int H, int G, float scale,
-                                                               int window, int keep_first, const float* sinks) {
+                                                               int window, int keep_first, const float* sinks,
+                                                               const float* gate, int64_t ldg) {
     constexpr int D = KS * 32, DV = CT * 16, SK = D + 8, SV = DV + 8;
     __shared__ __attribute__((aligned(16))) uint16_t Ks[64][SK];
     // values as pairs of neighbouring keys: dword [i][c] = V[2i][c] | V[2i+1][c] << 16, which is how the matrix
@@ -1310,8 +1419,13 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
             inv = expf(m - mn) / (l * expf(m - mn) + expf(sk - mn));
         }
         uint16_t* op = out + (int64_t)(start + myq) * ldo + (int64_t)h * DV + 4 * qd;
+        const float* gp = gate ? gate + (int64_t)(start + myq) * ldg + (int64_t)h * DV + 4 * qd : nullptr;
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct) {
+            if (gp) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) o[ct][j] *= sigmoid_f(gp[16 * ct + j]);
+            }
             uint2 w;
             w.x = pack_bf16x2(o[ct][0] * inv, o[ct][1] * inv);
             w.y = pack_bf16x2(o[ct][2] * inv, o[ct][3] * inv);
@@ -1324,8 +1438,8 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
 template <bool F32>
 __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float* y, int64_t ldy, const float* gate,
                                                                     int64_t ldg, const float* w, void* out_,
-                                                                    int64_t ldo, int n, int groups, int gate_first,
-                                                                    float eps) {
+                                                                    int64_t ldo, int n, int groups, int mode,
+                                                                    int w_shared, float eps) {
     typedef typename ActS<F32>::T T;
     __shared__ float red[4];
     T* out = (T*)out_;
@@ -1334,14 +1448,14 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
     const float* gr = gate + (int64_t)row * ldg + (int64_t)g * gs;
     float ss = 0.f;
     for (int c = threadIdx.x; c < gs; c += 256) {
-        const float u = gate_first ? yr[c] * silu_f(gr[c]) : yr[c];
+        const float u = mode == 1 ? yr[c] * silu_f(gr[c]) : yr[c];
         ss += u * u;
     }
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)gs + eps);
     for (int c = threadIdx.x; c < gs; c += 256) {
-        float u = gate_first ? (yr[c] * silu_f(gr[c])) * inv : (yr[c] * inv) * silu_f(gr[c]);
-        if (w) u *= w[g * gs + c];
+        float u = mode == 1 ? (yr[c] * silu_f(gr[c])) * inv : (yr[c] * inv) * (mode == 2 ? sigmoid_f(gr[c]) : silu_f(gr[c]));
+        if (w) u *= w[w_shared ? c : g * gs + c];
         ActS<F32>::st(out + (int64_t)row * ldo + (int64_t)g * gs + c, u);
     }
 }
@@ -1587,23 +1701,23 @@ int mv_rotary_pairs(float* x, int64_t ld, const double* inv_freq, const int32_t*
 }
 
 int mv_gated_group_norm(const float* y, int64_t ldy, const float* gate, int64_t ldg, const float* w, void* out,
-                        int64_t ldo, int rows, int n, int groups, int gate_first, float eps, int f32,
+                        int64_t ldo, int rows, int n, int groups, int mode, int w_shared, float eps, int f32,
                         mv_stream_t stream) {
     using namespace mv;
-    if (rows < 0 || n <= 0 || groups <= 0 || n % groups) return MV_ERR_INVALID_ARG;
+    if (rows < 0 || n <= 0 || groups <= 0 || n % groups || mode < 0 || mode > 2) return MV_ERR_INVALID_ARG;
     if (rows == 0) return MV_OK;
     if (!y || !gate || !out || ldy < n || ldg < n || ldo < n) return MV_ERR_INVALID_ARG;
     const int64_t units = (int64_t)rows * groups;
     hipStream_t s = (hipStream_t)stream;
     if (n / groups >= 1024) {
         const dim3 wide((unsigned)units);
-        if (f32) hipLaunchKernelGGL(gated_group_norm_wide_kernel<true>, wide, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, n, groups, gate_first, eps);
-        else hipLaunchKernelGGL(gated_group_norm_wide_kernel<false>, wide, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, n, groups, gate_first, eps);
+        if (f32) hipLaunchKernelGGL(gated_group_norm_wide_kernel<true>, wide, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, n, groups, mode, w_shared, eps);
+        else hipLaunchKernelGGL(gated_group_norm_wide_kernel<false>, wide, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, n, groups, mode, w_shared, eps);
         return check_launch();
     }
     const dim3 grid((unsigned)((units + 3) / 4));
-    if (f32) hipLaunchKernelGGL(gated_group_norm_kernel<true>, grid, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, rows, n, groups, gate_first, eps);
-    else hipLaunchKernelGGL(gated_group_norm_kernel<false>, grid, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, rows, n, groups, gate_first, eps);
+    if (f32) hipLaunchKernelGGL(gated_group_norm_kernel<true>, grid, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, rows, n, groups, mode, w_shared, eps);
+    else hipLaunchKernelGGL(gated_group_norm_kernel<false>, grid, dim3(256), 0, s, y, ldy, gate, ldg, w, out, ldo, rows, n, groups, mode, w_shared, eps);
     return check_launch();
 }
 
@@ -1653,6 +1767,28 @@ int mv_qk_rotary_store(float* qk, int64_t ld, const float* q_bias, const float* 
     return check_launch();
 }
 
+int mv_qkv_norm_rotary_store(float* qkv, int64_t ld, const float* q_bias, const float* k_bias, const float* v_bias,
+                             const float* q_norm, const float* k_norm, float eps, const double* inv_freq,
+                             float* v_first, int mix, float lam, void* k_cache, void* v_cache, const int32_t* tok_row,
+                             const int32_t* tok_pos, const int32_t* block_table, int bt_stride, int page, int tokens,
+                             int heads, int kv_heads, int d, int dv, int rot, int adjacent, int f32,
+                             mv_stream_t stream) {
+    using namespace mv;
+    if (tokens < 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || d <= 0 || dv <= 0 || page <= 0 || rot < 0 ||
+        rot > d || rot % 2 || rot > 8192 || mix < 0 || mix > 2)
+        return MV_ERR_INVALID_ARG;
+    if (tokens == 0) return MV_OK;
+    if (!qkv || ld < (int64_t)(heads + kv_heads) * d + (int64_t)kv_heads * dv || !k_cache || !v_cache || !tok_row ||
+        !tok_pos || !block_table || (rot > 0 && !inv_freq) || (mix && !v_first))
+        return MV_ERR_INVALID_ARG;
+    PagedRows pr{tok_row, tok_pos, block_table, bt_stride, page};
+    const size_t lds = (size_t)(rot > 0 ? rot : 1) * sizeof(float);
+    hipStream_t s = (hipStream_t)stream;
+    if (f32) hipLaunchKernelGGL(qkv_norm_rotary_store_kernel<true>, dim3(tokens), dim3(256), lds, s, qkv, ld, q_bias, k_bias, v_bias, q_norm, k_norm, eps, inv_freq, v_first, mix, lam, k_cache, v_cache, pr, heads, kv_heads, d, dv, rot, adjacent);
+    else hipLaunchKernelGGL(qkv_norm_rotary_store_kernel<false>, dim3(tokens), dim3(256), lds, s, qkv, ld, q_bias, k_bias, v_bias, q_norm, k_norm, eps, inv_freq, v_first, mix, lam, k_cache, v_cache, pr, heads, kv_heads, d, dv, rot, adjacent);
+    return check_launch();
+}
+
 int mv_window_attn_splits(int tokens, int heads, int kv_heads, int window, int keep_first) {
     using namespace mv;
     if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || window <= 0 || keep_first < 0) return 1;
@@ -1671,8 +1807,9 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
                    int page, const float* slopes, int tokens, int heads, int kv_heads, int d, int dv, float scale,
                    int window, int f32, const int32_t* row_len, const int32_t* ch_start, const int32_t* ch_len,
                    int chunks, int max_len, int keep_first, const float* sinks, float* part, int splits,
-                   int short_tokens, mv_stream_t stream) {
+                   int short_tokens, const float* gate, int64_t ldg, mv_stream_t stream) {
     using namespace mv;
+    if (gate && ldg < (int64_t)heads * dv) return MV_ERR_INVALID_ARG;
     if (tokens < 0 || heads <= 0 || kv_heads <= 0 || d <= 0 || dv <= 0 || page <= 0 || window <= 0 ||
         heads % kv_heads || keep_first < 0)
         return MV_ERR_INVALID_ARG;
@@ -1693,7 +1830,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
 #define MV_WA_TILE(KS_, CT_)                                                                                         \
     hipLaunchKernelGGL((window_attn_tile_kernel<KS_, CT_>), tg, dim3(256), 0, s, q, ldq, (const uint16_t*)k_cache,      \
                        (const uint16_t*)v_cache, (uint16_t*)out, ldo, pr, ch_start, ch_len, slopes, heads, kv_heads, scale, \
-                       window, keep_first, sinks);                                                                                    \
+                       window, keep_first, sinks, gate, ldg);                                                                         \
     skip_len = max_len
         if (d == 64 && dv == 64) { MV_WA_TILE(2, 4); }
         else if (d == 96 && dv == 96) { MV_WA_TILE(3, 6); }
@@ -1718,7 +1855,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
 #define MV_WA_GROUP(F32_, RT_)                                                                                         \
     hipLaunchKernelGGL((window_attn_group_kernel<F32_, RT_>), gg, dim3(256), glds, s, q, ldq, k_cache, v_cache, out, ldo, \
                        part, pr, slopes, sinks, heads, kv_heads, d, dv, scale, window, keep_first, row_len, skip_len,   \
-                       splits, vec)
+                       splits, vec, gate, ldg)
             if (f32) {
                 if (rt == 1) MV_WA_GROUP(true, 1); else if (rt == 2) MV_WA_GROUP(true, 2);
                 else if (rt == 4) MV_WA_GROUP(true, 4); else MV_WA_GROUP(true, 8);
@@ -1728,8 +1865,8 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
             }
 #undef MV_WA_GROUP
             if (splits > 1) {
-                if (f32) hipLaunchKernelGGL(window_attn_merge_kernel<true>, grid, dim3(64), 0, s, part, out, ldo, tok_row, sinks, heads, dv, splits, row_len, skip_len);
-                else hipLaunchKernelGGL(window_attn_merge_kernel<false>, grid, dim3(64), 0, s, part, out, ldo, tok_row, sinks, heads, dv, splits, row_len, skip_len);
+                if (f32) hipLaunchKernelGGL(window_attn_merge_kernel<true>, grid, dim3(64), 0, s, part, out, ldo, tok_row, sinks, heads, dv, splits, row_len, skip_len, gate, ldg);
+                else hipLaunchKernelGGL(window_attn_merge_kernel<false>, grid, dim3(64), 0, s, part, out, ldo, tok_row, sinks, heads, dv, splits, row_len, skip_len, gate, ldg);
             }
             return check_launch();
         }
@@ -1740,11 +1877,11 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
     const size_t lds = (size_t)(d + 64 * nw + 2 * nw + nw * dv) * sizeof(float);
     if (lds > 64 * 1024) return MV_ERR_UNSUPPORTED;
     if (wide) {
-        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks);
-        else hipLaunchKernelGGL((window_attn_kernel<false, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks);
+        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
+        else hipLaunchKernelGGL((window_attn_kernel<false, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
     } else {
-        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks);
-        else hipLaunchKernelGGL((window_attn_kernel<false, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks);
+        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
+        else hipLaunchKernelGGL((window_attn_kernel<false, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
     }
     return check_launch();
 }

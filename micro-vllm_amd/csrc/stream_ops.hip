@@ -2,10 +2,11 @@
 // sublayers in 32 bits and hand every projection a copy in the activation type (bf16, or fp32 when
 // the whole model runs in 32 bits).
 //
-//   embed_scaled:        x = table[id] * scale                       (fp32), h = act(x)
+//   embed_scaled:        x = table[id] * scale                       (fp32), h = act(x), or act of a norm of x
 //   postnorm_residual:   v = s1*y1 (+ s2*y2); x += v / sqrt(mean(v^2) + eps) * (1 + w); h = act(x)
 //                        (the norm sits on the SUBLAYER'S OUTPUT, its weight is stored as an offset
-//                        from one)
+//                        from one); optionally a bias inside v, a factor on what is added, and h = act of the NEXT
+//                        sublayer's norm of the new x
 //   offset_rmsnorm_gather: out = act( x[idx] / sqrt(mean(x[idx]^2) + eps) * (1 + w) )
 //   relu_squared:        out = act( max(v, 0)^2 )
 //   softcap:             v = cap * tanh(v / cap)
@@ -50,45 +51,150 @@ template <> struct Act<false> {
     static __device__ __forceinline__ void st(uint16_t* p, float v) { *p = (uint16_t)f32_to_bf16_bits(v); }
 };
 
+// w != NULL: h receives x / sqrt(mean(x^2) + eps) * (offset + w), the first layer's norm, instead of x itself
 template <bool F32>
 __global__ __launch_bounds__(256) void embed_scaled_kernel(const void* table_, const int* ids, float* x, int64_t ldx,
-                                                           void* h_, int64_t ldh, int n, int vocab, float scale) {
+                                                           void* h_, int64_t ldh, int n, int vocab, float scale,
+                                                           const float* w, float eps, float offset) {
     typedef typename Act<F32>::T T;
+    __shared__ float red[4];
     const T* table = (const T*)table_;
     T* h = (T*)h_;
     const int row = blockIdx.x;
     int id = ids[row];
     id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    float ss = 0.f;
     for (int c = threadIdx.x; c < n; c += 256) {
         const float v = Act<F32>::ld(table + (int64_t)id * n + c) * scale;
         x[(int64_t)row * ldx + c] = v;
-        Act<F32>::st(h + (int64_t)row * ldh + c, v);
-    }
-}
-
-template <bool F32>
-__global__ __launch_bounds__(256) void postnorm_residual_kernel(const float* y1, int64_t ld1, const float* y2,
-                                                                int64_t ld2, float s1, float s2, const float* w,
-                                                                float eps, float* x, int64_t ldx, void* h_,
-                                                                int64_t ldh, int n) {
-    typedef typename Act<F32>::T T;
-    __shared__ float red[4];
-    T* h = (T*)h_;
-    const int row = blockIdx.x;
-    const float* a = y1 + (int64_t)row * ld1;
-    const float* b = y2 ? y2 + (int64_t)row * ld2 : nullptr;
-    float ss = 0.f;
-    for (int c = threadIdx.x; c < n; c += 256) {
-        const float v = b ? s1 * a[c] + s2 * b[c] : s1 * a[c];
+        if (!w) Act<F32>::st(h + (int64_t)row * ldh + c, v);
         ss += v * v;
     }
+    if (!w) return;
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)n + eps);
     for (int c = threadIdx.x; c < n; c += 256) {
-        const float v = b ? s1 * a[c] + s2 * b[c] : s1 * a[c];
-        const float s = x[(int64_t)row * ldx + c] + (v * inv) * (1.0f + w[c]);
-        x[(int64_t)row * ldx + c] = s;
-        Act<F32>::st(h + (int64_t)row * ldh + c, s);
+        const float v = Act<F32>::ld(table + (int64_t)id * n + c) * scale;
+        Act<F32>::st(h + (int64_t)row * ldh + c, (v * inv) * (offset + w[c]));
+    }
+}
+
+struct PostnormArgs {
+    const float *y1, *y2, *bias, *w, *w2;
+    int64_t ld1, ld2, ldx, ldh;
+    float s1, s2, eps, mult;
+    float* x;
+    void* h;
+    int n;
+};
+
+template <bool F32>
+__global__ __launch_bounds__(256) void postnorm_residual_kernel(PostnormArgs a) {
+    typedef typename Act<F32>::T T;
+    __shared__ float red[4];
+    T* h = (T*)a.h;
+    const int row = blockIdx.x;
+    const float* y1 = a.y1 + (int64_t)row * a.ld1;
+    const float* y2 = a.y2 ? a.y2 + (int64_t)row * a.ld2 : nullptr;
+    auto value = [&](int c) {
+        float v = y2 ? a.s1 * y1[c] + a.s2 * y2[c] : a.s1 * y1[c];
+        return a.bias ? v + a.bias[c] : v;
+    };
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < a.n; c += 256) {
+        const float v = value(c);
+        ss += v * v;
+    }
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)a.n + a.eps);
+    float* xr = a.x + (int64_t)row * a.ldx;
+    float s2 = 0.f;
+    for (int c = threadIdx.x; c < a.n; c += 256) {
+        const float s = xr[c] + a.mult * ((value(c) * inv) * (1.0f + a.w[c]));
+        xr[c] = s;
+        if (!a.w2) Act<F32>::st(h + (int64_t)row * a.ldh + c, s);
+        s2 += s * s;
+    }
+    if (!a.w2) return;
+    s2 = block_sum(s2, red);
+    const float inv2 = 1.0f / sqrtf(s2 / (float)a.n + a.eps);
+    for (int c = threadIdx.x; c < a.n; c += 256)
+        Act<F32>::st(h + (int64_t)row * a.ldh + c, (xr[c] * inv2) * (1.0f + a.w2[c]));
+}
+
+// the same with the row in registers: n a multiple of 4 up to 1024 * NV, every row 16-byte aligned
+template <bool F32, int NV>
+__global__ __launch_bounds__(256) void postnorm_residual_reg_kernel(PostnormArgs a) {
+    __shared__ float red[4];
+    const int row = blockIdx.x, tid = threadIdx.x, n4 = a.n / 4;
+    const float4* y1 = reinterpret_cast<const float4*>(a.y1 + (int64_t)row * a.ld1);
+    const float4* y2 = a.y2 ? reinterpret_cast<const float4*>(a.y2 + (int64_t)row * a.ld2) : nullptr;
+    const float4* bias = reinterpret_cast<const float4*>(a.bias);
+    const float4* w = reinterpret_cast<const float4*>(a.w);
+    const float4* w2 = reinterpret_cast<const float4*>(a.w2);
+    float4* xr = reinterpret_cast<float4*>(a.x + (int64_t)row * a.ldx);
+    float4 v[NV], xv[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = tid + 256 * i;
+        v[i] = xv[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (c < n4) {
+            const float4 p = y1[c];
+            v[i] = make_float4(a.s1 * p.x, a.s1 * p.y, a.s1 * p.z, a.s1 * p.w);
+            if (y2) {
+                const float4 q = y2[c];
+                v[i].x += a.s2 * q.x; v[i].y += a.s2 * q.y; v[i].z += a.s2 * q.z; v[i].w += a.s2 * q.w;
+            }
+            if (bias) {
+                const float4 q = bias[c];
+                v[i].x += q.x; v[i].y += q.y; v[i].z += q.z; v[i].w += q.w;
+            }
+            xv[i] = xr[c];
+        }
+        ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+    }
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)a.n + a.eps);
+    float s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = tid + 256 * i;
+        if (c < n4) {
+            const float4 q = w[c];
+            xv[i].x += a.mult * ((v[i].x * inv) * (1.0f + q.x));
+            xv[i].y += a.mult * ((v[i].y * inv) * (1.0f + q.y));
+            xv[i].z += a.mult * ((v[i].z * inv) * (1.0f + q.z));
+            xv[i].w += a.mult * ((v[i].w * inv) * (1.0f + q.w));
+            xr[c] = xv[i];
+        }
+        s2 += xv[i].x * xv[i].x + xv[i].y * xv[i].y + xv[i].z * xv[i].z + xv[i].w * xv[i].w;
+    }
+    float inv2 = 1.0f;
+    if (a.w2) {
+        s2 = block_sum(s2, red);
+        inv2 = 1.0f / sqrtf(s2 / (float)a.n + a.eps);
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = tid + 256 * i;
+        if (c >= n4) continue;
+        float4 o = xv[i];
+        if (a.w2) {
+            const float4 q = w2[c];
+            o.x = (o.x * inv2) * (1.0f + q.x);
+            o.y = (o.y * inv2) * (1.0f + q.y);
+            o.z = (o.z * inv2) * (1.0f + q.z);
+            o.w = (o.w * inv2) * (1.0f + q.w);
+        }
+        if (F32) {
+            reinterpret_cast<float4*>((float*)a.h + (int64_t)row * a.ldh)[c] = o;
+        } else {
+            uint2 pk;
+            pk.x = pack_bf16x2(o.x, o.y);
+            pk.y = pack_bf16x2(o.z, o.w);
+            reinterpret_cast<uint2*>((uint16_t*)a.h + (int64_t)row * a.ldh)[c] = pk;
+        }
     }
 }
 
@@ -412,27 +518,46 @@ __global__ __launch_bounds__(256) void scale_kernel(float* v, int64_t count, flo
 extern "C" {
 
 int mv_embed_scaled(const void* table, const int32_t* ids, float* x, int64_t ldx, void* h, int64_t ldh, int rows,
-                    int n, int vocab, float scale, int f32, mv_stream_t stream) {
+                    int n, int vocab, float scale, const float* norm_w, float eps, float offset, int f32,
+                    mv_stream_t stream) {
     using namespace mv;
     if (rows < 0 || n <= 0 || vocab <= 0) return MV_ERR_INVALID_ARG;
     if (rows == 0) return MV_OK;
     if (!table || !ids || !x || !h || ldx < n || ldh < n) return MV_ERR_INVALID_ARG;
     hipStream_t s = (hipStream_t)stream;
-    if (f32) hipLaunchKernelGGL(embed_scaled_kernel<true>, dim3(rows), dim3(256), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale);
-    else hipLaunchKernelGGL(embed_scaled_kernel<false>, dim3(rows), dim3(256), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale);
+    if (f32) hipLaunchKernelGGL(embed_scaled_kernel<true>, dim3(rows), dim3(256), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale, norm_w, eps, offset);
+    else hipLaunchKernelGGL(embed_scaled_kernel<false>, dim3(rows), dim3(256), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale, norm_w, eps, offset);
     return check_launch();
 }
 
 int mv_postnorm_residual(const float* y1, int64_t ld1, const float* y2, int64_t ld2, float s1, float s2,
-                         const float* w, float eps, float* x, int64_t ldx, void* h, int64_t ldh, int rows, int n,
-                         int f32, mv_stream_t stream) {
+                         const float* bias, const float* w, float eps, float mult, const float* next_w, float* x,
+                         int64_t ldx, void* h, int64_t ldh, int rows, int n, int f32, mv_stream_t stream) {
     using namespace mv;
     if (rows < 0 || n <= 0) return MV_ERR_INVALID_ARG;
     if (rows == 0) return MV_OK;
     if (!y1 || !w || !x || !h || ld1 < n || (y2 && ld2 < n) || ldx < n || ldh < n) return MV_ERR_INVALID_ARG;
     hipStream_t s = (hipStream_t)stream;
-    if (f32) hipLaunchKernelGGL(postnorm_residual_kernel<true>, dim3(rows), dim3(256), 0, s, y1, ld1, y2, ld2, s1, s2, w, eps, x, ldx, h, ldh, n);
-    else hipLaunchKernelGGL(postnorm_residual_kernel<false>, dim3(rows), dim3(256), 0, s, y1, ld1, y2, ld2, s1, s2, w, eps, x, ldx, h, ldh, n);
+    PostnormArgs a;
+    a.y1 = y1; a.y2 = y2; a.bias = bias; a.w = w; a.w2 = next_w;
+    a.ld1 = ld1; a.ld2 = ld2; a.ldx = ldx; a.ldh = ldh;
+    a.s1 = s1; a.s2 = s2; a.eps = eps; a.mult = mult;
+    a.x = x; a.h = h; a.n = n;
+    const bool even = n % 4 == 0 && ld1 % 4 == 0 && ldx % 4 == 0 && ldh % 4 == 0 && (!y2 || ld2 % 4 == 0) && aligned16(y1) &&
+                      aligned16(x) && aligned16(h) && aligned16(w) && (!y2 || aligned16(y2)) &&
+                      (!bias || aligned16(bias)) && (!next_w || aligned16(next_w));
+#define MV_POSTNORM(NV_)                                                                                              \
+    do {                                                                                                              \
+        if (f32) hipLaunchKernelGGL((postnorm_residual_reg_kernel<true, NV_>), dim3(rows), dim3(256), 0, s, a);        \
+        else hipLaunchKernelGGL((postnorm_residual_reg_kernel<false, NV_>), dim3(rows), dim3(256), 0, s, a);           \
+    } while (0)
+    if (even && n <= 1024) MV_POSTNORM(1);
+    else if (even && n <= 2048) MV_POSTNORM(2);
+    else if (even && n <= 4096) MV_POSTNORM(4);
+    else if (even && n <= 8192) MV_POSTNORM(8);
+    else if (f32) hipLaunchKernelGGL(postnorm_residual_kernel<true>, dim3(rows), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(postnorm_residual_kernel<false>, dim3(rows), dim3(256), 0, s, a);
+#undef MV_POSTNORM
     return check_launch();
 }
 

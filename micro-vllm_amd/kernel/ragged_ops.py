@@ -75,23 +75,31 @@ class AnyLinear:
         return out
 
 
-def embed_scaled(table, ids, scale: float, x, h):
+def embed_scaled(table, ids, scale: float, x, h, w=None, eps: float = 0.0, offset: float = 1.0):
+    """x = table[ids] * scale; h = act(x), or with `w` act(x / sqrt(mean(x^2) + eps) * (offset + w))."""
     rows, n = x.shape
+    assert w is None or (w.numel() == n and w.is_contiguous())
     assert table.is_cuda and table.is_contiguous() and table.shape[1] == n and h.shape == x.shape
     assert table.dtype == h.dtype and ids.numel() == rows
     nv.check("mv_embed_scaled", nv.lib().mv_embed_scaled(
         table.data_ptr(), _i32(ids).data_ptr(), _f32(x).data_ptr(), _ld(x), h.data_ptr(), _ld(h), rows, n,
-        table.shape[0], float(scale), _is_f32(h), nv.stream_ptr()))
+        table.shape[0], float(scale), None if w is None else _f32(w).data_ptr(), float(eps), float(offset), _is_f32(h),
+        nv.stream_ptr()))
 
 
-def postnorm_residual(y1, w, eps: float, x, h, y2=None, s1: float = 1.0, s2: float = 0.0):
-    """x += unit_rms(s1*y1 + s2*y2) * (1 + w); h = x in the activation type."""
+def postnorm_residual(y1, w, eps: float, x, h, y2=None, s1: float = 1.0, s2: float = 0.0, bias=None, mult: float = 1.0,
+                      next_w=None):
+    """x += mult * unit_rms(s1*y1 + s2*y2 + bias) * (1 + w); h = x in the activation type, or with `next_w` the next
+    sublayer's norm of it, unit_rms(x) * (1 + next_w)."""
     rows, n = x.shape
+    assert bias is None or (bias.numel() == n and bias.is_contiguous())
+    assert next_w is None or (next_w.numel() == n and next_w.is_contiguous())
     assert y1.shape == (rows, n) and h.shape == (rows, n) and w.numel() == n and w.is_contiguous()
     assert y2 is None or y2.shape == (rows, n)
     nv.check("mv_postnorm_residual", nv.lib().mv_postnorm_residual(
         _f32(y1).data_ptr(), _ld(y1), None if y2 is None else _f32(y2).data_ptr(), 0 if y2 is None else _ld(y2),
-        float(s1), float(s2), _f32(w).data_ptr(), float(eps), _f32(x).data_ptr(), _ld(x), h.data_ptr(), _ld(h),
+        float(s1), float(s2), None if bias is None else _f32(bias).data_ptr(), _f32(w).data_ptr(), float(eps), float(mult),
+        None if next_w is None else _f32(next_w).data_ptr(), _f32(x).data_ptr(), _ld(x), h.data_ptr(), _ld(h),
         rows, n, _is_f32(h), nv.stream_ptr()))
 
 
@@ -198,13 +206,16 @@ def rotary_pairs_(x, inv_freq, tok_pos, heads: int, dim: int, rot: int, scale: f
         float(scale), nv.stream_ptr()))
 
 
-def gated_group_norm(y, gate, w, out, groups: int, gate_first: bool, eps: float):
+def gated_group_norm(y, gate, w, out, groups: int, gate_first: bool, eps: float, sigmoid: bool = False):
+    """Unit-RMS per group with a gate: silu(gate) before it (`gate_first`), silu(gate) or, with `sigmoid`, sigmoid(gate)
+    behind it; w of n values, or of n / groups values shared by all groups, multiplies last."""
     rows, n = y.shape
-    assert gate.shape == (rows, n) and out.shape == (rows, n) and n % groups == 0
-    assert w is None or (w.numel() == n and w.is_contiguous())
+    assert gate.shape == (rows, n) and out.shape == (rows, n) and n % groups == 0 and not (gate_first and sigmoid)
+    assert w is None or (w.numel() in (n, n // groups) and w.is_contiguous())
     nv.check("mv_gated_group_norm", nv.lib().mv_gated_group_norm(
         _f32(y).data_ptr(), _ld(y), _f32(gate).data_ptr(), _ld(gate), None if w is None else _f32(w).data_ptr(),
-        out.data_ptr(), _ld(out), rows, n, groups, int(gate_first), float(eps), _is_f32(out), nv.stream_ptr()))
+        out.data_ptr(), _ld(out), rows, n, groups, 2 if sigmoid else int(gate_first),
+        int(w is not None and w.numel() != n), float(eps), _is_f32(out), nv.stream_ptr()))
 
 
 def qk_unitnorm_store(qkv, k_cache, v_cache, step, heads: int, kv_heads: int, d: int, dv: int, eps: float):
@@ -253,13 +264,15 @@ def qk_rotary_store(qk, q_bias, k_bias, k_cache, v_cache, inv_freq, step, heads:
 
 
 def window_attn(q, k_cache, v_cache, out, step, slopes, heads: int, kv_heads: int, d: int, dv: int,
-                scale: float, window: int, tiled: bool = True, keep_first: int = 0, sinks=None, part=None, splits: int = 0):
+                scale: float, window: int, tiled: bool = True, keep_first: int = 0, sinks=None, part=None, splits: int = 0,
+                gate=None):
     """`tiled`: rows of more than SCAN_SEQ_MAX tokens go to the matrix-core kernel where it applies (bf16,
     the head shapes it is built for); False keeps every token on the plain kernel.  `keep_first`: positions below it
     stay visible behind the window; `sinks` [heads]: exp(sink) joins each head's denominator.  `part` (fp32, at least
     tokens * heads * splits * (dv + 2) values, `splits` from window_attn_splits): the tokens the matrix-core kernel
     does not take run the kernel that reads every key once for all query heads of its key/value head and cuts the keys
-    into `splits` pieces."""
+    into `splits` pieces.  `gate` [tokens, heads * dv] fp32: the output is multiplied by its sigmoid."""
+    assert gate is None or gate.shape == (q.shape[0], heads * dv)
     assert part is None or (splits >= 1 and part.is_contiguous() and part.numel() >= q.shape[0] * heads * splits * (dv + 2))
     assert sinks is None or (sinks.numel() == heads and sinks.is_contiguous())
     tokens = q.shape[0]
@@ -276,7 +289,8 @@ def window_attn(q, k_cache, v_cache, out, step, slopes, heads: int, kv_heads: in
         step.ch_start.data_ptr() if step.n_chunks else None, step.ch_len.data_ptr() if step.n_chunks else None,
         step.n_chunks if tiled else 0, SCAN_SEQ_MAX, int(keep_first), None if sinks is None else _f32(sinks).data_ptr(),
         None if part is None else _f32(part).data_ptr(), int(splits) if part is not None else 0,
-        int(getattr(step, "short_tokens", -1)) if tiled else -1, nv.stream_ptr()))
+        int(getattr(step, "short_tokens", -1)) if tiled else -1, None if gate is None else _f32(gate).data_ptr(),
+        0 if gate is None else _ld(gate), nv.stream_ptr()))
 
 
 def window_attn_splits(tokens: int, heads: int, kv_heads: int, window: int, keep_first: int = 0) -> int:
@@ -728,3 +742,79 @@ def gated_act_scaled(a, out, kind: int, scale, order=None, limit: float = 0.0, s
     nv.check("mv_gated_act_scaled", nv.lib().mv_gated_act_scaled(
         _f32(a).data_ptr(), _ld(a), out.data_ptr(), _ld(out), rows, n, int(kind), float(limit), float(slope),
         _f32(scale).data_ptr(), None if order is None else _i32(order).data_ptr(), _is_f32(out), nv.stream_ptr()))
+
+
+# ---------------------------------------------------------------------------------------------------------
+# Norm over whole projections with mixed values, delta-rule memory (csrc/seq_mix.hip, delta.hip)
+
+def qkv_norm_rotary_store(qkv, k_cache, v_cache, step, heads: int, kv_heads: int, d: int, dv: int, inv_freq, rot: int,
+                          eps: float, q_bias=None, k_bias=None, v_bias=None, q_norm=None, k_norm=None, v_first=None,
+                          mix: int = 0, lam: float = 0.0, adjacent: bool = False):
+    """qkv [T, heads*d + kv_heads*(d + dv)] fp32 = q | k | v of one projection.  q and k get their biases, an RMS norm over
+    all heads at once (weights q_norm / k_norm; None: no norm) and the rotation of each head's first `rot` dimensions; q
+    stays in place, k goes to its page.  v gets its bias; mix 1 keeps it in v_first [T, kv_heads*dv], mix 2 blends
+    (1 - lam) v + lam v_first; it goes to its page."""
+    tokens = qkv.shape[0]
+    page = k_cache.shape[1]
+    assert qkv.shape[1] == (heads + kv_heads) * d + kv_heads * dv and step.tokens == tokens
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dtype == v_cache.dtype
+    assert k_cache.shape[1:] == (page, kv_heads, d) and v_cache.shape == (k_cache.shape[0], page, kv_heads, dv)
+    assert int(step.max_page) < k_cache.shape[0] and page == step.page
+    for t, n in ((q_bias, heads * d), (k_bias, kv_heads * d), (v_bias, kv_heads * dv), (q_norm, heads * d),
+                 (k_norm, kv_heads * d)):
+        assert t is None or (t.numel() == n and t.is_contiguous())
+    assert rot == 0 or (inv_freq.is_cuda and inv_freq.dtype == torch.float64 and inv_freq.numel() == rot // 2)
+    assert mix in (0, 1, 2) and (mix == 0 or (v_first.shape == (tokens, kv_heads * dv) and v_first.is_contiguous()))
+    p = lambda t: None if t is None else _f32(t).data_ptr()   # noqa: E731
+    nv.check("mv_qkv_norm_rotary_store", nv.lib().mv_qkv_norm_rotary_store(
+        _f32(qkv).data_ptr(), _ld(qkv), p(q_bias), p(k_bias), p(v_bias), p(q_norm), p(k_norm), float(eps),
+        None if rot == 0 else inv_freq.data_ptr(), p(v_first) if mix else None, int(mix), float(lam), k_cache.data_ptr(),
+        v_cache.data_ptr(), step.tok_row.data_ptr(), step.tok_pos.data_ptr(), step.block_table.data_ptr(),
+        step.block_table.stride(0), page, tokens, heads, kv_heads, d, dv, rot, int(adjacent), _is_f32(k_cache),
+        nv.stream_ptr()))
+
+
+def delta_prep(proj, state, wt, out, beta, low, step, kv_heads: int, n: int, heads: int, p: int, b_off: int, low_off: int,
+               eps: float):
+    """proj [T, ...] fp32 = q | k | v (| ... head logits at b_off, low-rank columns at low_off): short convolutions
+    (wt [taps, C] fp32, state [slots, taps - 1, C] fp32) with SiLU into out [T, C], unit length per head of q (times
+    n^-1/2) and k, beta = sigmoid(logits), low = the low-rank columns in the activation type."""
+    tokens, C = out.shape
+    taps, low_n = wt.shape[0], low.shape[1]
+    assert C == 2 * kv_heads * n + heads * p and wt.shape[1] == C and wt.is_contiguous() and step.tokens == tokens
+    assert proj.shape[0] == tokens and proj.shape[1] >= max(b_off + heads, low_off + low_n) and b_off >= C and low_off >= C
+    assert state.is_contiguous() and state.shape[1:] == (max(taps - 1, 0), C) and int(step.max_slot) < state.shape[0]
+    assert beta.shape == (tokens, heads) and beta.is_contiguous() and low.shape[0] == tokens
+    nv.check("mv_delta_prep", nv.lib().mv_delta_prep(
+        _f32(proj).data_ptr(), _ld(proj), b_off, low_off, low_n, _f32(state).data_ptr(), _f32(wt).data_ptr(),
+        _f32(out).data_ptr(), _ld(out), _f32(beta).data_ptr(), low.data_ptr(), _ld(low), step.tok_row.data_ptr(),
+        step.row_start.data_ptr(), step.row_len.data_ptr(), step.row_ctx.data_ptr(), step.row_slot.data_ptr(), tokens,
+        step.rows, kv_heads, n, heads, p, taps, float(eps), n ** -0.5, _is_f32(low), nv.stream_ptr()))
+
+
+def delta_rule(qkv, gate_in, z, beta, dt_bias, a_log, norm, state, out, step, kv_heads: int, heads: int, n: int, p: int,
+               eps: float, chunked: bool = True):
+    """The delta-rule recurrence of delta_prep's q | k | v with gates exp(-exp(a_log) softplus(gate_in + dt_bias)) per
+    state row; out [T, heads*p] = act(unit-RMS per head * norm * sigmoid(z)); state [slots, heads, n, p] fp32.  Rows of
+    up to SCAN_SEQ_MAX tokens run token by token; longer rows in chunks of 64 unless `chunked` is False or the head's
+    shape does not fit a workgroup's LDS."""
+    tokens = qkv.shape[0]
+    assert qkv.shape[1] == 2 * kv_heads * n + heads * p and gate_in.shape == (tokens, heads * n)
+    assert z.shape == (tokens, heads * p) and out.shape == (tokens, heads * p) and beta.shape == (tokens, heads)
+    assert beta.is_contiguous() and dt_bias.numel() == heads * n and dt_bias.is_contiguous() and a_log.numel() == heads
+    assert norm.numel() == p and norm.is_contiguous() and step.tokens == tokens
+    assert state.is_contiguous() and state.shape[1:] == (heads, n, p) and int(step.max_slot) < state.shape[0]
+    L = nv.lib()
+    chunks = step.n_chunks if chunked and L.mv_delta_chunked_ok(n, p) else 0
+    scratch = None
+    if chunks:
+        scratch = torch.empty(chunks * heads * L.mv_delta_scratch_floats(n, p), dtype=torch.float32, device=qkv.device)
+    nv.check("mv_delta_rule", L.mv_delta_rule(
+        _f32(qkv).data_ptr(), _ld(qkv), _f32(gate_in).data_ptr(), _ld(gate_in), _f32(z).data_ptr(), _ld(z),
+        _f32(beta).data_ptr(), _f32(dt_bias).data_ptr(), _f32(a_log).data_ptr(), _f32(norm).data_ptr(),
+        _f32(state).data_ptr(), out.data_ptr(), _ld(out), step.row_start.data_ptr(), step.row_len.data_ptr(),
+        step.row_ctx.data_ptr(), step.row_slot.data_ptr(), step.rows, kv_heads, heads, n, p, float(eps),
+        None if scratch is None else scratch.data_ptr(), step.ch_start.data_ptr() if chunks else None,
+        step.ch_len.data_ptr() if chunks else None, step.row_ch0.data_ptr() if chunks else None,
+        step.row_nch.data_ptr() if chunks else None, chunks, SCAN_SEQ_MAX,
+        int(getattr(step, "short_tokens", -1)) if chunks else -1, _is_f32(out), nv.stream_ptr()))
