@@ -95,6 +95,15 @@ def parse():
                          "with latent attention and routed experts - at equal width and depth; one JSON line of its own")
     ap.add_argument("--solopel-widths", default="1024,2048,4096")
     ap.add_argument("--solopel-kernels", action="store_true", help="with --solopel: per-op times of one step on stderr")
+    ap.add_argument("--dugazen", action="store_true",
+                    help="instead of the default workload: prefill and decode throughput of the Dugazen design "
+                         "(delta-rule memories with a decay per state row, windowed attention with norms over whole "
+                         "projections and mixed values, clamped feed-forwards; random weights) at a few widths beside "
+                         "the family's closest designs at equal width, depth and dense feed-forward parameters: Pagazen "
+                         "(state-space heads and windowed attention) and Fagunex (a gate per state row); one JSON "
+                         "line of its own")
+    ap.add_argument("--dugazen-widths", default="1024,2048,4096")
+    ap.add_argument("--dugazen-kernels", action="store_true", help="with --dugazen: per-op times of one step on stderr")
     return ap.parse_args()
 
 
@@ -766,6 +775,35 @@ def solopel_compare(args, dev):
                       "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "n_gpus": 1, "rows": rows}), flush=True)
 
 
+def dugazen_compare(args, dev):
+    """Prefill (one prompt of --ctx tokens) and decode (bs 1 and 8 at context --ctx) of the Dugazen design beside
+    Pagazen and Fagunex, all through InferenceEngine.run_ragged.  Random weights, 4 layers (3 recurrent + 1
+    attention each), vocabulary 32000, 128-wide heads.  Dugazen: 128 x 128 delta-rule states, low-rank maps of 128, a
+    window of 1024, feed-forwards of gate, up and down with 4 x width; Pagazen: 128 x 64 states, the same window, up
+    and down with 6 x width (the same feed-forward parameters); Fagunex: 128 x 128 gated states, latent attention,
+    routed experts with 4 x width active."""
+    import micro_vllm_amd  # noqa: F401
+    from micro_vllm_amd.core.engine import InferenceEngine
+    from micro_vllm_amd.models import dugazen, fagunex, pagazen
+
+    S, layers, rows = args.ctx, 4, []
+    for width in [int(w) for w in args.dugazen_widths.split(",")]:
+        row = {"width": width, "layers": layers, "ctx": S}
+        for name, make in (("dugazen", lambda: dugazen.build_random_model(dugazen.bench_config(width, layers), 1, rank=128)),
+                           ("pagazen", lambda: pagazen.build_random_model(pagazen.bench_config(width, layers, ff_mult=6), 1)),
+                           ("fagunex", lambda: fagunex.build_random_model(fagunex.bench_config(width, layers), 1))):
+            model = make()
+            eng = InferenceEngine(model=model, max_batch_size=8, max_prefill_tokens=S, n_blocks=9 * (S // 64 + 4),
+                                  max_tokens=S + 256, state_slots=9)
+            row.update(_ragged_engine_row(eng, model.config, S, name, args.dugazen_kernels, width))
+            del eng, model
+            torch.cuda.empty_cache()
+        log(f"[bench] {row}")
+        rows.append(row)
+    print(json.dumps({"metric": "Dugazen beside Pagazen and Fagunex (ragged family): prefill and decode tokens/s at equal size",
+                      "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "n_gpus": 1, "rows": rows}), flush=True)
+
+
 def pagazen_kernel_table(eng, ids, width):
     """Per-op time of one prefill step and one single-token step (rocprof-free: HIP events around each
     wrapper call), printed on stderr."""
@@ -778,7 +816,8 @@ def pagazen_kernel_table(eng, ids, width):
              "sigmoid_gate", "linear_heads", "linear_segments", "gate_lower_bound_", "scan_gated", "latent_prep",
              "latent_attn", "moe_route", "moe_plan", "moe_combine", "embed_pair", "add_rmsnorm", "rmsnorm_gather",
              "gated_act", "qk_rotary_store", "moe_route_scored", "gated_residual_norm", "cast_concat", "gelu_tanh",
-             "scale_", "conv_taps", "conv_qkv_store", "diff_attn", "moe_route_sigmoid", "gated_act_scaled"]
+             "scale_", "conv_taps", "conv_qkv_store", "diff_attn", "moe_route_sigmoid", "gated_act_scaled", "qkv_norm_rotary_store",
+             "delta_prep", "delta_rule"]
     saved = {n: getattr(ops, n) for n in names}
     saved_call = ops.AnyLinear.__call__
 
@@ -916,6 +955,9 @@ def main():
     if args.solopel:
         assert world == 1, "--solopel runs on one GPU"
         return solopel_compare(args, dev)
+    if args.dugazen:
+        assert world == 1, "--dugazen runs on one GPU"
+        return dugazen_compare(args, dev)
     peers = world > 1                 # ranks to synchronise with
     if args.as_rank_of:
         assert world == 1, "--as-rank-of runs one process"
