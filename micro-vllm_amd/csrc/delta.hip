@@ -100,6 +100,95 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a) {
     }
 }
 
+// The same for up to four taps: a wave takes TB neighbouring tokens of its unit and keeps their inputs in registers, so
+// that a token's row is read once instead of once per tap; NI: 64-channel groups of a unit (a head, or a stretch of v).
+template <bool F32, int NI, int TB>
+__global__ __launch_bounds__(256) void delta_prep4_kernel(DeltaPrepArgs a) {
+    const int lane = threadIdx.x & 63, unit = blockIdx.y;
+    const int vu = (a.H * a.p + 64 * NI - 1) / (64 * NI), units = 2 * a.K + vu + 1;
+    const int t0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * TB;
+    if (t0 >= a.T) return;
+    const int tn = a.T - t0 < TB ? a.T - t0 : TB;
+    if (unit == units - 1) {
+        for (int tb = 0; tb < tn; ++tb) {
+            const int64_t t = t0 + tb;
+            const float* row = a.proj + t * a.ldp;
+            for (int h = lane; h < a.H; h += 64) a.beta[t * a.H + h] = sigmoid_d(row[a.b_off + h]);
+            typename ActD<F32>::T* lo = (typename ActD<F32>::T*)a.low + t * a.ldl;
+            for (int c = lane; c < a.low_n; c += 64) ActD<F32>::st(lo + c, row[a.low_off + c]);
+        }
+        return;
+    }
+    const bool head = unit < 2 * a.K;
+    const int C = 2 * a.K * a.n + a.H * a.p;
+    const int c0 = head ? unit * a.n : 2 * a.K * a.n + (unit - 2 * a.K) * 64 * NI;
+    const int cnt = head ? a.n : (C - c0 < 64 * NI ? C - c0 : 64 * NI);
+    const int keep = a.taps - 1, skip = 4 - a.taps;
+    float w[NI][4], x[NI][TB + 3];
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+        const int cl = lane + 64 * i;
+        const bool ok = cl < cnt;
+        const float* col = a.proj + c0 + (ok ? cl : 0);
+#pragma unroll
+        for (int s = 0; s < TB + 3; ++s) {
+            const int ft = t0 - 3 + s;
+            x[i][s] = (ok && ft >= 0 && ft < a.T) ? col[(int64_t)ft * a.ldp] : 0.f;
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) w[i][j] = (ok && j >= skip) ? a.wt[(int64_t)(j - skip) * C + c0 + cl] : 0.f;
+    }
+#pragma unroll
+    for (int tb = 0; tb < TB; ++tb) {
+        if (tb >= tn) break;
+        const int t = t0 + tb, b = a.r.tok_row[t], rel = t - a.r.row_start[b];
+        float y[NI], ss = 0.f;
+        if (rel >= 3 && !a.in_place) {
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                float acc = 0.f;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc = fmaf(w[i][j], x[i][tb + j], acc);
+                y[i] = acc;
+            }
+        } else {
+            // the row's first tokens: inputs from before the step lie in the slot
+            const bool carried = a.r.row_ctx[b] > 0;
+            float* st = a.state + (int64_t)a.r.row_slot[b] * keep * C + c0;
+            float v[NI][4];
+#pragma unroll
+            for (int i = 0; i < NI; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const int src = rel - 3 + j, cl = lane + 64 * i;
+                    v[i][j] = x[i][tb + j];
+                    if (src < 0) v[i][j] = (carried && j >= skip && cl < cnt) ? st[(int64_t)(src + keep) * C + cl] : 0.f;
+                }
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                float acc = 0.f;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc = fmaf(w[i][j], v[i][j], acc);
+                y[i] = acc;
+                if (a.in_place && lane + 64 * i < cnt)
+#pragma unroll
+                    for (int j = 1; j < 4; ++j)
+                        if (j > skip) st[(int64_t)(j - skip - 1) * C + lane + 64 * i] = v[i][j];
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            y[i] *= sigmoid_d(y[i]);
+            ss += y[i] * y[i];
+        }
+        float f = 1.0f;
+        if (head) f = (1.0f / sqrtf(wave_sum(ss) + a.eps)) * (unit < a.K ? a.qscale : 1.0f);
+#pragma unroll
+        for (int i = 0; i < NI; ++i)
+            if (lane + 64 * i < cnt) a.out[(int64_t)t * a.ldo + c0 + lane + 64 * i] = y[i] * f;
+    }
+}
+
 // keeps each row's last taps - 1 inputs (rows of any length; used when some row has more than one token)
 __global__ __launch_bounds__(256) void delta_conv_state_kernel(DeltaPrepArgs a, int B) {
     const int C = 2 * a.K * a.n + a.H * a.p, keep = a.taps - 1;
@@ -246,8 +335,9 @@ constexpr int kDCh = 64;
 // scratch per (chunk, head): qd [64][n16], wk [64][n16], kt [n16][64], uv [64][p16], bm [64][64], s0 [n16][p16], gc [n16]
 __device__ __forceinline__ int pad16(int v) { return (v + 15) & ~15; }
 
-template <int DUMMY>
-__global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
+constexpr int kIntra = 512;      // threads of the intra kernel: two waves a SIMD, one workgroup a compute unit
+
+__global__ __launch_bounds__(kIntra) void delta_chunk_intra_kernel(DeltaArgs a) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int ch = blockIdx.y, h = blockIdx.x, tid = threadIdx.x;
     const int wv = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
@@ -262,64 +352,74 @@ __global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
     const int start = a.ch_start[ch], len = a.ch_len[ch], kh = h / (a.H / a.K);
     const int64_t unit = (int64_t)ch * a.H + h;
     const float neg_a = -expf(a.a_log[h]);
-    for (int i = tid; i < kDCh * N; i += 256) {
-        const int t = i / N, c = i - t * N;
-        float q_ = 0.f, k_ = 0.f, g_ = 1.f;
-        if (t < len && c < n) {
-            const float* qp = a.qkv + (int64_t)(start + t) * a.ldq + (int64_t)kh * n + c;
-            q_ = qp[0];
-            k_ = qp[(int64_t)a.K * n];
-            g_ = decay_gate(a.a[(int64_t)(start + t) * a.lda + (int64_t)h * n + c], a.dt_bias[(int64_t)h * n + c], neg_a);
+    constexpr int kB = 8;            // loads in flight together (addresses clamped, values selected afterwards)
+    for (int i0 = tid; i0 < kDCh * N; i0 += kIntra * kB) {
+        float q_[kB], k_[kB], a_[kB], b_[kB];
+#pragma unroll
+        for (int u = 0; u < kB; ++u) {
+            const int i = i0 + kIntra * u, t = i / N, c = i - t * N;
+            const int64_t tok = start + (t < len ? t : len - 1);
+            const int cc = c < n ? c : n - 1;
+            const float* qp = a.qkv + tok * a.ldq + (int64_t)kh * n + cc;
+            q_[u] = qp[0];
+            k_[u] = qp[(int64_t)a.K * n];
+            a_[u] = a.a[tok * a.lda + (int64_t)h * n + cc];
+            b_[u] = a.dt_bias[(int64_t)h * n + cc];
         }
-        Q[t * SN + c] = q_;
-        Kp[t * SN + c] = k_;
-        Gn[t * SN + c] = g_;
+#pragma unroll
+        for (int u = 0; u < kB; ++u) {
+            const int i = i0 + kIntra * u, t = i / N, c = i - t * N;
+            if (t >= kDCh) continue;
+            const bool ok = t < len && c < n;
+            Q[t * SN + c] = ok ? q_[u] : 0.f;
+            Kp[t * SN + c] = ok ? k_[u] : 0.f;
+            Gn[t * SN + c] = ok ? decay_gate(a_[u], b_[u], neg_a) : 1.f;
+        }
     }
     if (tid < kDCh) bs[tid] = tid < len ? a.beta[(int64_t)(start + tid) * a.H + h] : 0.f;
     __syncthreads();
-    // the diagonal block of the wave: lane (r, g) holds column s = r, state rows 16 m + 4 g .. + 3
+    // diagonal blocks, A by the first four waves and B by the others: lane (r, g) holds column s = r, state rows
+    // 16 m + 4 g .. + 3
     {
-        float sa[16], sb[16];
+        const int blk = wv & 3;
+        const bool isb = wv >= 4;
+        float sa[16];
 #pragma unroll
-        for (int t = 0; t < 16; ++t) sa[t] = sb[t] = 0.f;
-        const float* q0 = Q + 16 * wv * SN + 4 * g;
-        const float* k0 = Kp + 16 * wv * SN + 4 * g;
-        const float* g0 = Gn + 16 * wv * SN + 4 * g;
+        for (int t = 0; t < 16; ++t) sa[t] = 0.f;
+        const float* l0 = (isb ? Q : Kp) + 16 * blk * SN + 4 * g;
+        const float* k0 = Kp + 16 * blk * SN + 4 * g;
+        const float* g0 = Gn + 16 * blk * SN + 4 * g;
         for (int m = 0; m < N; m += 16) {
             const float4 ks = *reinterpret_cast<const float4*>(k0 + r * SN + m);
             float4 w = make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll
             for (int t = 0; t < 16; ++t) {
                 const float4 gt = *reinterpret_cast<const float4*>(g0 + t * SN + m);
-                const float4 kt = *reinterpret_cast<const float4*>(k0 + t * SN + m);
-                const float4 qt = *reinterpret_cast<const float4*>(q0 + t * SN + m);
+                const float4 lt = *reinterpret_cast<const float4*>(l0 + t * SN + m);
                 const bool self = t == r;
                 w.x = self ? ks.x : w.x * gt.x;
                 w.y = self ? ks.y : w.y * gt.y;
                 w.z = self ? ks.z : w.z * gt.z;
                 w.w = self ? ks.w : w.w * gt.w;
-                sa[t] = fmaf(kt.x, w.x, fmaf(kt.y, w.y, fmaf(kt.z, w.z, fmaf(kt.w, w.w, sa[t]))));
-                sb[t] = fmaf(qt.x, w.x, fmaf(qt.y, w.y, fmaf(qt.z, w.z, fmaf(qt.w, w.w, sb[t]))));
+                sa[t] = fmaf(lt.x, w.x, fmaf(lt.y, w.y, fmaf(lt.z, w.z, fmaf(lt.w, w.w, sa[t]))));
             }
         }
         float* bm = a.bm + unit * (kDCh * kDCh);
 #pragma unroll
         for (int t = 0; t < 16; ++t) {
-            float x = sa[t], y = sb[t];
+            float x = sa[t];
             x += __shfl_xor(x, 16, 64);
             x += __shfl_xor(x, 32, 64);
-            y += __shfl_xor(y, 16, 64);
-            y += __shfl_xor(y, 32, 64);
             if ((t >> 2) == g) {
-                const int tt = 16 * wv + t;
-                Am[tt * 68 + 16 * wv + r] = r < t ? -bs[tt] * x : 0.f;
-                bm[tt * kDCh + 16 * wv + r] = r <= t ? y : 0.f;
+                const int tt = 16 * blk + t;
+                if (isb) bm[tt * kDCh + 16 * blk + r] = r <= t ? x : 0.f;
+                else Am[tt * 68 + 16 * blk + r] = r < t ? -bs[tt] * x : 0.f;
             }
         }
     }
     __syncthreads();
     // products of the gates, in place: thread per (block, state row)
-    for (int i = tid; i < 4 * N; i += 256) {
+    for (int i = tid; i < 4 * N; i += kIntra) {
         const int blk = i / N, c = i - blk * N;
         float* qc = Q + 16 * blk * SN + c;
         float* kc = Kp + 16 * blk * SN + c;
@@ -345,8 +445,8 @@ __global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
         }
         E[blk * N + c] = pre;
     }
-    // inverse of the wave's unit triangular diagonal block: lane r owns column r, forward substitution
-    if (g == 0) {
+    // inverses of the unit triangular diagonal blocks: lane r owns column r, forward substitution
+    if (wv < 4 && g == 0) {
         float x[16];
         const float* m = Am + (16 * wv) * 68 + 16 * wv;
 #pragma unroll
@@ -359,9 +459,9 @@ __global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
         }
     }
     __syncthreads();
-    // blocks below the diagonal: six block pairs, A and B each, three products a wave
-    for (int x = 0; x < 3; ++x) {
-        const int id = wv * 3 + x, pair = id >> 1;
+    // blocks below the diagonal: six block pairs, A and B each
+    for (int id = wv; id < 12; id += kIntra / 64) {
+        const int pair = id >> 1;
         const bool isb = id & 1;
         const int I = pair == 0 ? 1 : (pair < 3 ? 2 : 3), J = pair == 0 ? 0 : (pair < 3 ? pair - 1 : pair - 3);
         f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -391,28 +491,36 @@ __global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
     }
     // operands of the other two kernels
     float* qd = a.qd + unit * (kDCh * N);
-    for (int i = tid; i < kDCh * N; i += 256) {
+    for (int i = tid; i < kDCh * N; i += kIntra) {
         const int t = i / N, c = i - t * N;
         float v = Q[t * SN + c];
         for (int M = 0; M < (t >> 4); ++M) v *= E[M * N + c];
         qd[i] = v;
     }
     float* kt = a.kt + unit * (kDCh * N);
-    for (int i = tid; i < kDCh * N; i += 256) {
+    for (int i = tid; i < kDCh * N; i += kIntra) {
         const int c = i >> 6, s = i & 63;
         float v = Gn[s * SN + c];
         for (int M = (s >> 4) + 1; M < 4; ++M) v *= E[M * N + c];
         kt[i] = v;
     }
-    for (int c = tid; c < N; c += 256) a.gc[unit * N + c] = ((E[c] * E[N + c]) * E[2 * N + c]) * E[3 * N + c];
+    for (int c = tid; c < N; c += kIntra) a.gc[unit * N + c] = ((E[c] * E[N + c]) * E[2 * N + c]) * E[3 * N + c];
     __syncthreads();
     // the triangular system, 16 columns at a time: first those of V, then those of G * K
     const int pt = P / 16, ntile = pt + N / 16;
     float* uv = a.uv + unit * (kDCh * P);
     float* wk = a.wk + unit * (kDCh * N);
-    for (int tile = wv; tile < ntile; tile += 4) {
+    for (int tile = wv; tile < ntile; tile += kIntra / 64) {
         const bool isv = tile < pt;
         const int c = 16 * (isv ? tile : tile - pt) + r;
+        float vv[16];
+        if (isv) {
+#pragma unroll
+            for (int i = 0; i < 16; ++i) {
+                const int t = 16 * (i >> 2) + 4 * g + (i & 3);
+                vv[i] = a.qkv[(int64_t)(start + (t < len ? t : len - 1)) * a.ldq + (int64_t)2 * a.K * n + (int64_t)h * p + (c < p ? c : p - 1)];
+            }
+        }
         f32x4_t X[4];
         float e = 1.f;           // product of the blocks before I for column c of G * K
 #pragma unroll
@@ -422,7 +530,7 @@ __global__ __launch_bounds__(256) void delta_chunk_intra_kernel(DeltaArgs a) {
             for (int j = 0; j < 4; ++j) {
                 const int t = 16 * I + 4 * g + j;
                 float v;
-                if (isv) v = (t < len && c < p) ? a.qkv[(int64_t)(start + t) * a.ldq + (int64_t)2 * a.K * n + (int64_t)h * p + c] : 0.f;
+                if (isv) v = (t < len && c < p) ? vv[4 * I + j] : 0.f;
                 else v = Kp[t * SN + c] * e;
                 acc[j] = bs[t] * v;
             }
@@ -477,47 +585,52 @@ __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
         }
     }
     const int64_t u0 = (int64_t)a.row_ch0[b] * a.H + h;
-    float4 wk[NT], kt[OWN][4], gm[OWN];
-    f32x4_t uv;
-    auto fetch = [&](int64_t unit) {
+    struct Operands {
+        float4 wk[NT], kt[OWN][4], gm[OWN];
+        f32x4_t uv;
+    };
+    auto fetch = [&](int64_t unit, Operands& x) {
         const float* w = a.wk + unit * (kDCh * N) + (16 * wv + r) * N + 4 * g;
 #pragma unroll
         for (int i = 0; i < NT; ++i)
-            if (i < nt) wk[i] = *reinterpret_cast<const float4*>(w + 16 * i);
+            if (i < nt) x.wk[i] = *reinterpret_cast<const float4*>(w + 16 * i);
 #pragma unroll
         for (int o = 0; o < OWN; ++o) {
             const int it = wv + 4 * o;
             if (it < nt) {
                 const float* k = a.kt + unit * (kDCh * N) + (16 * it + r) * kDCh + 4 * g;
 #pragma unroll
-                for (int t = 0; t < 4; ++t) kt[o][t] = *reinterpret_cast<const float4*>(k + 16 * t);
-                gm[o] = *reinterpret_cast<const float4*>(a.gc + unit * N + 16 * it + 4 * g);
+                for (int t = 0; t < 4; ++t) x.kt[o][t] = *reinterpret_cast<const float4*>(k + 16 * t);
+                x.gm[o] = *reinterpret_cast<const float4*>(a.gc + unit * N + 16 * it + 4 * g);
             }
         }
         const float* up = a.uv + unit * (kDCh * P) + (16 * wv + 4 * g) * P + c0 + r;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) uv[j] = up[j * P];
+        for (int j = 0; j < 4; ++j) x.uv[j] = up[j * P];
     };
-    fetch(u0);
+    Operands cur, nxt;
+    fetch(u0, cur);
+    nxt = cur;
     __syncthreads();
     for (int c = 0; c < nch; ++c) {
         const int64_t unit = u0 + (int64_t)c * a.H;
+        if (c + 1 < nch) fetch(unit + a.H, nxt);     // under way while this chunk is worked on
         // two accumulators: neighbouring products do not wait for each other
         f32x4_t x0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, x1 = x0;
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
             if (i < nt) {
                 const int k = 16 * i + 4 * g;
-                MV_DMFMA(x0, wk[i].x, Ss[k][r]);
-                MV_DMFMA(x1, wk[i].y, Ss[k + 1][r]);
-                MV_DMFMA(x0, wk[i].z, Ss[k + 2][r]);
-                MV_DMFMA(x1, wk[i].w, Ss[k + 3][r]);
+                MV_DMFMA(x0, cur.wk[i].x, Ss[k][r]);
+                MV_DMFMA(x1, cur.wk[i].y, Ss[k + 1][r]);
+                MV_DMFMA(x0, cur.wk[i].z, Ss[k + 2][r]);
+                MV_DMFMA(x1, cur.wk[i].w, Ss[k + 3][r]);
             }
         }
         float* up = a.uv + unit * (kDCh * P) + (16 * wv + 4 * g) * P + c0 + r;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const float u = uv[j] - (x0[j] + x1[j]);
+            const float u = cur.uv[j] - (x0[j] + x1[j]);
             Us[16 * wv + 4 * g + j][r] = u;
             up[j * P] = u;
         }
@@ -535,15 +648,15 @@ __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
         for (int o = 0; o < OWN; ++o) {
             const int it = wv + 4 * o;
             if (it >= nt) continue;
-            f32x4_t y0 = f32x4_t{S[o][0] * gm[o].x, S[o][1] * gm[o].y, S[o][2] * gm[o].z, S[o][3] * gm[o].w};
+            f32x4_t y0 = f32x4_t{S[o][0] * cur.gm[o].x, S[o][1] * cur.gm[o].y, S[o][2] * cur.gm[o].z, S[o][3] * cur.gm[o].w};
             f32x4_t y1 = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
                 const int k = 16 * t + 4 * g;
-                MV_DMFMA(y0, kt[o][t].x, Us[k][r]);
-                MV_DMFMA(y1, kt[o][t].y, Us[k + 1][r]);
-                MV_DMFMA(y0, kt[o][t].z, Us[k + 2][r]);
-                MV_DMFMA(y1, kt[o][t].w, Us[k + 3][r]);
+                MV_DMFMA(y0, cur.kt[o][t].x, Us[k][r]);
+                MV_DMFMA(y1, cur.kt[o][t].y, Us[k + 1][r]);
+                MV_DMFMA(y0, cur.kt[o][t].z, Us[k + 2][r]);
+                MV_DMFMA(y1, cur.kt[o][t].w, Us[k + 3][r]);
             }
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
@@ -551,8 +664,8 @@ __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
                 Ss[16 * it + 4 * g + j][r] = S[o][j];
             }
         }
-        if (c + 1 < nch) fetch(unit + a.H);
         __syncthreads();
+        cur = nxt;
     }
 #pragma unroll
     for (int o = 0; o < OWN; ++o)
@@ -663,11 +776,27 @@ int mv_delta_prep(const float* proj, int64_t ldp, int b_off, int low_off, int lo
     a.in_place = tokens == rows && taps > 1;       // every row has one token
     a.eps = eps; a.qscale = q_scale;
     hipStream_t s = (hipStream_t)stream;
-    const int units = 2 * kv_heads + (heads * p + 255) / 256 + 1;
+    const int ni = n <= 64 ? 1 : n <= 128 ? 2 : n <= 256 ? 4 : 8;
+    const int vw = taps <= 4 ? 64 * ni : 256;
+    const int units = 2 * kv_heads + (heads * p + vw - 1) / vw + 1;
     if (units > 65535) return MV_ERR_UNSUPPORTED;
-    const dim3 grid((tokens + 3) / 4, units);
-    if (f32) hipLaunchKernelGGL(delta_prep_kernel<true>, grid, dim3(256), 0, s, a);
-    else hipLaunchKernelGGL(delta_prep_kernel<false>, grid, dim3(256), 0, s, a);
+    if (taps <= 4) {
+        const int tb = tokens > 64 ? 4 : 1;
+        const dim3 grid((tokens + 4 * tb - 1) / (4 * tb), units);
+#define MV_PREP4(NI_)                                                                                                  \
+    do {                                                                                                               \
+        if (f32 && tb == 4) hipLaunchKernelGGL((delta_prep4_kernel<true, NI_, 4>), grid, dim3(256), 0, s, a);            \
+        else if (f32) hipLaunchKernelGGL((delta_prep4_kernel<true, NI_, 1>), grid, dim3(256), 0, s, a);                  \
+        else if (tb == 4) hipLaunchKernelGGL((delta_prep4_kernel<false, NI_, 4>), grid, dim3(256), 0, s, a);             \
+        else hipLaunchKernelGGL((delta_prep4_kernel<false, NI_, 1>), grid, dim3(256), 0, s, a);                          \
+    } while (0)
+        if (ni == 1) MV_PREP4(1); else if (ni == 2) MV_PREP4(2); else if (ni == 4) MV_PREP4(4); else MV_PREP4(8);
+#undef MV_PREP4
+    } else {
+        const dim3 grid((tokens + 3) / 4, units);
+        if (f32) hipLaunchKernelGGL(delta_prep_kernel<true>, grid, dim3(256), 0, s, a);
+        else hipLaunchKernelGGL(delta_prep_kernel<false>, grid, dim3(256), 0, s, a);
+    }
     if (taps > 1 && !a.in_place) {
         const int64_t work = (int64_t)rows * C;
         hipLaunchKernelGGL(delta_conv_state_kernel, dim3((unsigned)((work + 255) / 256)), dim3(256), 0, s, a, rows);
@@ -742,8 +871,8 @@ int mv_delta_rule(const float* qkv, int64_t ldq, const float* gate_in, int64_t l
         a.gc = a.s0 + U * N * P;
         const size_t lds1 = delta_intra_lds(n), lds2 = (size_t)kDCh * (P + 4) * sizeof(float);
         static LdsOptIn o1, o2[2][4];
-        if (int rc = ensure_dynamic_lds((const void*)delta_chunk_intra_kernel<0>, lds1, o1)) return rc;
-        hipLaunchKernelGGL(delta_chunk_intra_kernel<0>, dim3(heads, chunks), dim3(256), lds1, s, a);
+        if (int rc = ensure_dynamic_lds((const void*)delta_chunk_intra_kernel, lds1, o1)) return rc;
+        hipLaunchKernelGGL(delta_chunk_intra_kernel, dim3(heads, chunks), dim3(kIntra), lds1, s, a);
         const dim3 gc(heads, (unsigned)(P / 16), rows);
         if (N <= 32) hipLaunchKernelGGL(delta_chunk_carry_kernel<2>, gc, dim3(256), 0, s, a);
         else if (N <= 64) hipLaunchKernelGGL(delta_chunk_carry_kernel<4>, gc, dim3(256), 0, s, a);

@@ -699,7 +699,7 @@ __global__ __launch_bounds__(256) void qk_rotary_store_kernel(float* qk, int64_t
 // place, k goes to the key page.  v gets its bias; mix 1: v is kept in vfirst [T, G * dv]; mix 2: v = (1 - lam) v + lam
 // vfirst; v goes to the value page.
 template <bool F32>
-__global__ __launch_bounds__(256) void qkv_norm_rotary_store_kernel(float* qkv, int64_t ld, const float* qb,
+__global__ __launch_bounds__(1024) void qkv_norm_rotary_store_kernel(float* qkv, int64_t ld, const float* qb,
                                                                     const float* kb, const float* vb, const float* qn,
                                                                     const float* kn, float eps, const double* inv_freq,
                                                                     float* vfirst, int mix, float lam, void* kc_,
@@ -707,17 +707,17 @@ __global__ __launch_bounds__(256) void qkv_norm_rotary_store_kernel(float* qkv, 
                                                                     int dv, int rot, int adjacent) {
     typedef typename ActS<F32>::T T_;
     extern __shared__ float ang[];     // [rot / 2] cosines, then sines
-    __shared__ float red[8];
+    __shared__ float red[32];
     T_* kc = (T_*)kc_;
     T_* vc = (T_*)vc_;
-    const int t = blockIdx.x, tid = threadIdx.x, pos = pr.tok_pos[t];
+    const int t = blockIdx.x, tid = threadIdx.x, NT = blockDim.x, pos = pr.tok_pos[t];
     float* q = qkv + (int64_t)t * ld;
     float* k = q + (int64_t)H * d;
     const float* v = k + (int64_t)G * d;
     const int pg = pr.block_table[(int64_t)pr.tok_row[t] * pr.bt_stride + pos / pr.page];
     const int64_t slot = (int64_t)pg * pr.page + pos % pr.page;
     const int half = rot / 2;
-    for (int i = tid; i < half; i += 256) {
+    for (int i = tid; i < half; i += NT) {
         const double a = (double)pos * inv_freq[i];
         ang[i] = (float)cos(a);
         ang[half + i] = (float)sin(a);
@@ -725,14 +725,14 @@ __global__ __launch_bounds__(256) void qkv_norm_rotary_store_kernel(float* qkv, 
     float sq = 0.f, sk = 0.f;
     if (qn) {
 #pragma unroll 4
-        for (int c = tid; c < H * d; c += 256) {
+        for (int c = tid; c < H * d; c += NT) {
             const float x = qb ? q[c] + qb[c] : q[c];
             sq += x * x;
         }
     }
     if (kn) {
 #pragma unroll 4
-        for (int c = tid; c < G * d; c += 256) {
+        for (int c = tid; c < G * d; c += NT) {
             const float x = kb ? k[c] + kb[c] : k[c];
             sk += x * x;
         }
@@ -741,13 +741,18 @@ __global__ __launch_bounds__(256) void qkv_norm_rotary_store_kernel(float* qkv, 
     sk = wave_sum(sk);
     if ((tid & 63) == 0) {
         red[tid >> 6] = sq;
-        red[4 + (tid >> 6)] = sk;
+        red[16 + (tid >> 6)] = sk;
     }
     __syncthreads();
-    const float iq = qn ? 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)(H * d) + eps) : 1.f;
-    const float ik = kn ? 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)(G * d) + eps) : 1.f;
+    sq = sk = 0.f;
+    for (int i = 0; i < NT / 64; ++i) {
+        sq += red[i];
+        sk += red[16 + i];
+    }
+    const float iq = qn ? 1.0f / sqrtf(sq / (float)(H * d) + eps) : 1.f;
+    const float ik = kn ? 1.0f / sqrtf(sk / (float)(G * d) + eps) : 1.f;
     const int per = d - half;         // a head's items: `half` rotated pairs, then the dimensions behind them
-    for (int i = tid; i < (H + G) * per; i += 256) {
+    for (int i = tid; i < (H + G) * per; i += NT) {
         const int u = i / per, j = i - u * per;
         const bool isq = u < H;
         const int base = isq ? u * d : (u - H) * d;
@@ -779,7 +784,7 @@ __global__ __launch_bounds__(256) void qkv_norm_rotary_store_kernel(float* qkv, 
             else if (pg >= 0) ActS<F32>::st(kc + slot * G * d + c, x);
         }
     }
-    for (int c = tid; c < G * dv; c += 256) {
+    for (int c = tid; c < G * dv; c += NT) {
         float x = vb ? v[c] + vb[c] : v[c];
         float* f = mix ? vfirst + (int64_t)t * G * dv + c : nullptr;
         if (mix == 1) *f = x;
@@ -1783,9 +1788,10 @@ int mv_qkv_norm_rotary_store(float* qkv, int64_t ld, const float* q_bias, const 
         return MV_ERR_INVALID_ARG;
     PagedRows pr{tok_row, tok_pos, block_table, bt_stride, page};
     const size_t lds = (size_t)(rot > 0 ? rot : 1) * sizeof(float);
+    const int nt = tokens <= 512 ? 1024 : 256;      // a token of a short step has its workgroup to itself on a compute unit
     hipStream_t s = (hipStream_t)stream;
-    if (f32) hipLaunchKernelGGL(qkv_norm_rotary_store_kernel<true>, dim3(tokens), dim3(256), lds, s, qkv, ld, q_bias, k_bias, v_bias, q_norm, k_norm, eps, inv_freq, v_first, mix, lam, k_cache, v_cache, pr, heads, kv_heads, d, dv, rot, adjacent);
-    else hipLaunchKernelGGL(qkv_norm_rotary_store_kernel<false>, dim3(tokens), dim3(256), lds, s, qkv, ld, q_bias, k_bias, v_bias, q_norm, k_norm, eps, inv_freq, v_first, mix, lam, k_cache, v_cache, pr, heads, kv_heads, d, dv, rot, adjacent);
+    if (f32) hipLaunchKernelGGL(qkv_norm_rotary_store_kernel<true>, dim3(tokens), dim3(nt), lds, s, qkv, ld, q_bias, k_bias, v_bias, q_norm, k_norm, eps, inv_freq, v_first, mix, lam, k_cache, v_cache, pr, heads, kv_heads, d, dv, rot, adjacent);
+    else hipLaunchKernelGGL(qkv_norm_rotary_store_kernel<false>, dim3(tokens), dim3(nt), lds, s, qkv, ld, q_bias, k_bias, v_bias, q_norm, k_norm, eps, inv_freq, v_first, mix, lam, k_cache, v_cache, pr, heads, kv_heads, d, dv, rot, adjacent);
     return check_launch();
 }
 

@@ -53,18 +53,18 @@ template <> struct Act<false> {
 
 // w != NULL: h receives x / sqrt(mean(x^2) + eps) * (offset + w), the first layer's norm, instead of x itself
 template <bool F32>
-__global__ __launch_bounds__(256) void embed_scaled_kernel(const void* table_, const int* ids, float* x, int64_t ldx,
+__global__ __launch_bounds__(1024) void embed_scaled_kernel(const void* table_, const int* ids, float* x, int64_t ldx,
                                                            void* h_, int64_t ldh, int n, int vocab, float scale,
                                                            const float* w, float eps, float offset) {
     typedef typename Act<F32>::T T;
-    __shared__ float red[4];
+    __shared__ float red[16];
     const T* table = (const T*)table_;
     T* h = (T*)h_;
     const int row = blockIdx.x;
     int id = ids[row];
     id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
     float ss = 0.f;
-    for (int c = threadIdx.x; c < n; c += 256) {
+    for (int c = threadIdx.x; c < n; c += blockDim.x) {
         const float v = Act<F32>::ld(table + (int64_t)id * n + c) * scale;
         x[(int64_t)row * ldx + c] = v;
         if (!w) Act<F32>::st(h + (int64_t)row * ldh + c, v);
@@ -73,7 +73,7 @@ __global__ __launch_bounds__(256) void embed_scaled_kernel(const void* table_, c
     if (!w) return;
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)n + eps);
-    for (int c = threadIdx.x; c < n; c += 256) {
+    for (int c = threadIdx.x; c < n; c += blockDim.x) {
         const float v = Act<F32>::ld(table + (int64_t)id * n + c) * scale;
         Act<F32>::st(h + (int64_t)row * ldh + c, (v * inv) * (offset + w[c]));
     }
@@ -122,10 +122,10 @@ __global__ __launch_bounds__(256) void postnorm_residual_kernel(PostnormArgs a) 
         Act<F32>::st(h + (int64_t)row * a.ldh + c, (xr[c] * inv2) * (1.0f + a.w2[c]));
 }
 
-// the same with the row in registers: n a multiple of 4 up to 1024 * NV, every row 16-byte aligned
+// the same with the row in registers: n a multiple of 4 up to 4 * threads * NV, every row 16-byte aligned
 template <bool F32, int NV>
-__global__ __launch_bounds__(256) void postnorm_residual_reg_kernel(PostnormArgs a) {
-    __shared__ float red[4];
+__global__ __launch_bounds__(1024) void postnorm_residual_reg_kernel(PostnormArgs a) {
+    __shared__ float red[16];
     const int row = blockIdx.x, tid = threadIdx.x, n4 = a.n / 4;
     const float4* y1 = reinterpret_cast<const float4*>(a.y1 + (int64_t)row * a.ld1);
     const float4* y2 = a.y2 ? reinterpret_cast<const float4*>(a.y2 + (int64_t)row * a.ld2) : nullptr;
@@ -137,7 +137,7 @@ __global__ __launch_bounds__(256) void postnorm_residual_reg_kernel(PostnormArgs
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-        const int c = tid + 256 * i;
+        const int c = tid + (int)blockDim.x * i;
         v[i] = xv[i] = make_float4(0.f, 0.f, 0.f, 0.f);
         if (c < n4) {
             const float4 p = y1[c];
@@ -159,7 +159,7 @@ __global__ __launch_bounds__(256) void postnorm_residual_reg_kernel(PostnormArgs
     float s2 = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-        const int c = tid + 256 * i;
+        const int c = tid + (int)blockDim.x * i;
         if (c < n4) {
             const float4 q = w[c];
             xv[i].x += a.mult * ((v[i].x * inv) * (1.0f + q.x));
@@ -177,7 +177,7 @@ __global__ __launch_bounds__(256) void postnorm_residual_reg_kernel(PostnormArgs
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-        const int c = tid + 256 * i;
+        const int c = tid + (int)blockDim.x * i;
         if (c >= n4) continue;
         float4 o = xv[i];
         if (a.w2) {
@@ -447,6 +447,21 @@ __global__ __launch_bounds__(256) void gated_act_kernel(const float* a, int64_t 
     Act<F32>::st(out + row * ldo + c, gated_act_f(a[row * lda + c], a[row * lda + n + c], kind, limit, slope));
 }
 
+// four values a thread: n a multiple of 4, rows 16-byte aligned
+template <bool F32>
+__global__ __launch_bounds__(256) void gated_act4_kernel(const float* a, int64_t lda, void* out, int64_t ldo, int n,
+                                                         int kind, float limit, float slope) {
+    const int64_t row = blockIdx.x;
+    const int c = (blockIdx.y * 256 + threadIdx.x) * 4;
+    if (c >= n) return;
+    const float4 g = *reinterpret_cast<const float4*>(a + row * lda + c);
+    const float4 u = *reinterpret_cast<const float4*>(a + row * lda + n + c);
+    const float4 o = make_float4(gated_act_f(g.x, u.x, kind, limit, slope), gated_act_f(g.y, u.y, kind, limit, slope),
+                                 gated_act_f(g.z, u.z, kind, limit, slope), gated_act_f(g.w, u.w, kind, limit, slope));
+    if (F32) *reinterpret_cast<float4*>((float*)out + row * ldo + c) = o;
+    else *reinterpret_cast<uint2*>((uint16_t*)out + row * ldo + c) = make_uint2(pack_bf16x2(o.x, o.y), pack_bf16x2(o.z, o.w));
+}
+
 
 // mode 0: x as it is; 1: x += y * sigmoid(g + b); 2: x = y + b.  w != NULL: the norm of the new x, to n32 (fp32)
 // and / or h (activation type)
@@ -525,8 +540,9 @@ int mv_embed_scaled(const void* table, const int32_t* ids, float* x, int64_t ldx
     if (rows == 0) return MV_OK;
     if (!table || !ids || !x || !h || ldx < n || ldh < n) return MV_ERR_INVALID_ARG;
     hipStream_t s = (hipStream_t)stream;
-    if (f32) hipLaunchKernelGGL(embed_scaled_kernel<true>, dim3(rows), dim3(256), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale, norm_w, eps, offset);
-    else hipLaunchKernelGGL(embed_scaled_kernel<false>, dim3(rows), dim3(256), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale, norm_w, eps, offset);
+    const int nt = rows <= 512 && n > 1024 ? 1024 : 256;
+    if (f32) hipLaunchKernelGGL(embed_scaled_kernel<true>, dim3(rows), dim3(nt), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale, norm_w, eps, offset);
+    else hipLaunchKernelGGL(embed_scaled_kernel<false>, dim3(rows), dim3(nt), 0, s, table, ids, x, ldx, h, ldh, n, vocab, scale, norm_w, eps, offset);
     return check_launch();
 }
 
@@ -546,15 +562,17 @@ int mv_postnorm_residual(const float* y1, int64_t ld1, const float* y2, int64_t 
     const bool even = n % 4 == 0 && ld1 % 4 == 0 && ldx % 4 == 0 && ldh % 4 == 0 && (!y2 || ld2 % 4 == 0) && aligned16(y1) &&
                       aligned16(x) && aligned16(h) && aligned16(w) && (!y2 || aligned16(y2)) &&
                       (!bias || aligned16(bias)) && (!next_w || aligned16(next_w));
+    // a row of a short step has its workgroup to itself on a compute unit: more threads, fewer values each
+    const int nt = rows > 512 || n <= 1024 ? 256 : n <= 2048 ? 512 : 1024;
 #define MV_POSTNORM(NV_)                                                                                              \
     do {                                                                                                              \
-        if (f32) hipLaunchKernelGGL((postnorm_residual_reg_kernel<true, NV_>), dim3(rows), dim3(256), 0, s, a);        \
-        else hipLaunchKernelGGL((postnorm_residual_reg_kernel<false, NV_>), dim3(rows), dim3(256), 0, s, a);           \
+        if (f32) hipLaunchKernelGGL((postnorm_residual_reg_kernel<true, NV_>), dim3(rows), dim3(nt), 0, s, a);         \
+        else hipLaunchKernelGGL((postnorm_residual_reg_kernel<false, NV_>), dim3(rows), dim3(nt), 0, s, a);            \
     } while (0)
-    if (even && n <= 1024) MV_POSTNORM(1);
-    else if (even && n <= 2048) MV_POSTNORM(2);
-    else if (even && n <= 4096) MV_POSTNORM(4);
-    else if (even && n <= 8192) MV_POSTNORM(8);
+    if (even && n <= 4 * nt) MV_POSTNORM(1);
+    else if (even && n <= 8 * nt) MV_POSTNORM(2);
+    else if (even && n <= 16 * nt) MV_POSTNORM(4);
+    else if (even && n <= 32 * nt) MV_POSTNORM(8);
     else if (f32) hipLaunchKernelGGL(postnorm_residual_kernel<true>, dim3(rows), dim3(256), 0, s, a);
     else hipLaunchKernelGGL(postnorm_residual_kernel<false>, dim3(rows), dim3(256), 0, s, a);
 #undef MV_POSTNORM
@@ -611,8 +629,14 @@ int mv_gated_act(const float* a, int64_t lda, void* out, int64_t ldo, int rows, 
     if (rows < 0 || n <= 0 || kind < 0 || kind > 2) return MV_ERR_INVALID_ARG;
     if (rows == 0) return MV_OK;
     if (!a || !out || lda < 2 * (int64_t)n || ldo < n) return MV_ERR_INVALID_ARG;
-    const dim3 grid(rows, (n + 255) / 256);
     hipStream_t s = (hipStream_t)stream;
+    if (n % 4 == 0 && lda % 4 == 0 && ldo % 4 == 0 && aligned16(a) && aligned16(out)) {
+        const dim3 grid4(rows, (n / 4 + 255) / 256);
+        if (f32) hipLaunchKernelGGL(gated_act4_kernel<true>, grid4, dim3(256), 0, s, a, lda, out, ldo, n, kind, limit, slope);
+        else hipLaunchKernelGGL(gated_act4_kernel<false>, grid4, dim3(256), 0, s, a, lda, out, ldo, n, kind, limit, slope);
+        return check_launch();
+    }
+    const dim3 grid(rows, (n + 255) / 256);
     if (f32) hipLaunchKernelGGL(gated_act_kernel<true>, grid, dim3(256), 0, s, a, lda, out, ldo, n, kind, limit, slope);
     else hipLaunchKernelGGL(gated_act_kernel<false>, grid, dim3(256), 0, s, a, lda, out, ldo, n, kind, limit, slope);
     return check_launch();
