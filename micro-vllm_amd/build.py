@@ -57,9 +57,8 @@ FLAGS = [
     "-Wno-unused-function",
 ]
 
-# no packed fp32 arithmetic (v_pk_*_f32), the scalar forms only: for the sources that were written with
-# it.  The older sources keep the flags their kernels were tuned and tested with.
-_NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+# no packed fp32 arithmetic (v_pk_*_f32), the scalar forms only, in every source
+FLAGS += ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 # per-source additions.  attn_prefill.hip: the pipelined attention deals its vector work out slot
@@ -67,13 +66,6 @@ _NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 # into one chain of packed additions (slower beside MFMAs than the scalar form, and serial)
 FILE_FLAGS = {
     "attn_prefill.hip": ["-fno-slp-vectorize"],
-    "linear_any.hip": _NO_PACKED_F32,
-    "stream_ops.hip": _NO_PACKED_F32,
-    "seq_mix.hip": _NO_PACKED_F32,
-    "latent_attn.hip": _NO_PACKED_F32,
-    "moe.hip": _NO_PACKED_F32,
-    "diff_attn.hip": _NO_PACKED_F32,
-    "delta.hip": _NO_PACKED_F32,
 }
 
 

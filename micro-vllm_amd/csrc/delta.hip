@@ -23,7 +23,11 @@ template <> struct ActD<false> {
     static __device__ __forceinline__ void st(uint16_t* p, float v) { *p = (uint16_t)f32_to_bf16_bits(v); }
 };
 
-__device__ __forceinline__ float sigmoid_d(float v) { return 1.0f / (1.0f + expf(-v)); }
+constexpr float kLog2E = 1.4426950408889634f;
+// 1 / (1 + e^-v) on the hardware's 2^x and reciprocal (each within one unit in the last place)
+__device__ __forceinline__ float sigmoid_d(float v) {
+    return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-v * kLog2E));
+}
 
 struct DeltaRows {
     const int *tok_row, *row_start, *row_len, *row_ctx, *row_slot;
@@ -138,10 +142,15 @@ __global__ __launch_bounds__(256) void delta_prep4_kernel(DeltaPrepArgs a) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) w[i][j] = (ok && j >= skip) ? a.wt[(int64_t)(j - skip) * C + c0 + cl] : 0.f;
     }
+    int row[TB], at[TB];          // each token's row and its place there, looked up together
+#pragma unroll
+    for (int tb = 0; tb < TB; ++tb) row[tb] = a.r.tok_row[tb < tn ? t0 + tb : t0];
+#pragma unroll
+    for (int tb = 0; tb < TB; ++tb) at[tb] = t0 + tb - a.r.row_start[row[tb]];
 #pragma unroll
     for (int tb = 0; tb < TB; ++tb) {
         if (tb >= tn) break;
-        const int t = t0 + tb, b = a.r.tok_row[t], rel = t - a.r.row_start[b];
+        const int t = t0 + tb, b = row[tb], rel = at[tb];
         float y[NI], ss = 0.f;
         if (rel >= 3 && !a.in_place) {
 #pragma unroll
@@ -215,17 +224,29 @@ struct DeltaArgs {
     float* state;           // [slots, H, n, p]
     void* out;              // [T, ldo] activation type
     DeltaRows r;
-    int K, H, n, p, max_len;
+    int K, H, n, p, max_len, vec;
     float eps;
     // chunks of long rows
     const int *ch_start, *ch_len, *row_ch0, *row_nch;
     float *qd, *wk, *kt, *uv, *bm, *s0, *gc;     // scratch, see DeltaScratch
 };
 
+// exp(neg_a * softplus(raw + bias)).  softplus(v) = max(v, 0) + log(1 + e) with e = exp(-|v|), and
+// log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3, by its series to s^15 (the rest is below 2e-9 of the sum): the
+// relative precision stays where e is small - a gate next to one, applied a thousand times over.
 __device__ __forceinline__ float decay_gate(float raw, float bias, float neg_a) {
     const float v = raw + bias;
-    const float sp = fmaxf(v, 0.f) + log1pf(expf(-fabsf(v)));     // log(1 + e^v)
-    return expf(neg_a * sp);
+    const float e = __builtin_amdgcn_exp2f(-fabsf(v) * kLog2E);
+    const float s = e * __builtin_amdgcn_rcpf(2.0f + e), s2 = s * s;
+    float c = fmaf(s2, 1.0f / 15.0f, 1.0f / 13.0f);
+    c = fmaf(s2, c, 1.0f / 11.0f);
+    c = fmaf(s2, c, 1.0f / 9.0f);
+    c = fmaf(s2, c, 1.0f / 7.0f);
+    c = fmaf(s2, c, 1.0f / 5.0f);
+    c = fmaf(s2, c, 1.0f / 3.0f);
+    c = fmaf(s2, c, 1.0f);
+    const float sp = fmaf(2.0f * s, c, fmaxf(v, 0.f));
+    return __builtin_amdgcn_exp2f((neg_a * kLog2E) * sp);
 }
 
 // One workgroup per (head, row).  Thread (ng, cl) holds the state rows ng * npt .. + npt of column cl; columns are
@@ -332,7 +353,9 @@ __global__ void delta_scan_kernel(DeltaArgs a, int pw) {
 constexpr int kDCh = 64;
 #define MV_DMFMA(acc, a_, b_) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a_, b_, acc, 0, 0, 0)
 
-// scratch per (chunk, head): qd [64][n16], wk [64][n16], kt [n16][64], uv [64][p16], bm [64][64], s0 [n16][p16], gc [n16]
+// scratch per (chunk, head): qd, wk (64 x n16) and kt (n16 x 64) in the order in which the lanes of a wave read them as
+// operand A - tile by tile of 16 x 16, lane (r, g) holding row r, columns 4 g .. + 3 -, uv (64 x p16) and s0 (n16 x p16)
+// as slabs of 16 columns, bm [64][64], gc [n16]
 __device__ __forceinline__ int pad16(int v) { return (v + 15) & ~15; }
 
 constexpr int kIntra = 512;      // threads of the intra kernel: two waves a SIMD, one workgroup a compute unit
@@ -489,38 +512,53 @@ __global__ __launch_bounds__(kIntra) void delta_chunk_intra_kernel(DeltaArgs a) 
             else Am[t * 68 + s] = -bs[t] * acc[j];
         }
     }
-    // operands of the other two kernels
-    float* qd = a.qd + unit * (kDCh * N);
-    for (int i = tid; i < kDCh * N; i += kIntra) {
-        const int t = i / N, c = i - t * N;
-        float v = Q[t * SN + c];
-        for (int M = 0; M < (t >> 4); ++M) v *= E[M * N + c];
-        qd[i] = v;
-    }
-    float* kt = a.kt + unit * (kDCh * N);
-    for (int i = tid; i < kDCh * N; i += kIntra) {
-        const int c = i >> 6, s = i & 63;
-        float v = Gn[s * SN + c];
-        for (int M = (s >> 4) + 1; M < 4; ++M) v *= E[M * N + c];
-        kt[i] = v;
+    // the wave's first 16 columns of V are under way from here on
+    float vv[16];
+    auto load_v = [&](int tile) {
+        const int c = 16 * tile + r < p ? 16 * tile + r : p - 1;
+        const float* vp = a.qkv + (int64_t)2 * a.K * n + (int64_t)h * p + c;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int t = 16 * (i >> 2) + 4 * g + (i & 3);
+            vv[i] = vp[(int64_t)(start + (t < len ? t : len - 1)) * a.ldq];
+        }
+    };
+    if (wv < P / 16) load_v(wv);
+    // operands of the other two kernels, 16 x 16 tiles in operand order
+    const int nt = N / 16;
+    float4* qd = reinterpret_cast<float4*>(a.qd + unit * (kDCh * N));
+    float4* kt = reinterpret_cast<float4*>(a.kt + unit * (kDCh * N));
+    for (int i = tid; i < 16 * N; i += kIntra) {
+        const int rr = i & 15, gg = (i >> 4) & 3, tl = i >> 6;
+        {
+            const int blk = tl / nt, c = 16 * (tl - blk * nt) + 4 * gg;
+            float4 v = *reinterpret_cast<const float4*>(Q + (16 * blk + rr) * SN + c);
+            for (int M = 0; M < blk; ++M) {
+                const float4 e = *reinterpret_cast<const float4*>(E + M * N + c);
+                v.x *= e.x;
+                v.y *= e.y;
+                v.z *= e.z;
+                v.w *= e.w;
+            }
+            qd[i] = v;
+        }
+        {
+            const int blk = tl & 3, c = 16 * (tl >> 2) + rr;
+            const float* k4 = Gn + (16 * blk + 4 * gg) * SN + c;
+            float f = 1.f;
+            for (int M = blk + 1; M < 4; ++M) f *= E[M * N + c];
+            kt[i] = make_float4(k4[0] * f, k4[SN] * f, k4[2 * SN] * f, k4[3 * SN] * f);
+        }
     }
     for (int c = tid; c < N; c += kIntra) a.gc[unit * N + c] = ((E[c] * E[N + c]) * E[2 * N + c]) * E[3 * N + c];
     __syncthreads();
     // the triangular system, 16 columns at a time: first those of V, then those of G * K
     const int pt = P / 16, ntile = pt + N / 16;
     float* uv = a.uv + unit * (kDCh * P);
-    float* wk = a.wk + unit * (kDCh * N);
     for (int tile = wv; tile < ntile; tile += kIntra / 64) {
         const bool isv = tile < pt;
         const int c = 16 * (isv ? tile : tile - pt) + r;
-        float vv[16];
-        if (isv) {
-#pragma unroll
-            for (int i = 0; i < 16; ++i) {
-                const int t = 16 * (i >> 2) + 4 * g + (i & 3);
-                vv[i] = a.qkv[(int64_t)(start + (t < len ? t : len - 1)) * a.ldq + (int64_t)2 * a.K * n + (int64_t)h * p + (c < p ? c : p - 1)];
-            }
-        }
+        if (isv && tile != wv) load_v(tile);
         f32x4_t X[4];
         float e = 1.f;           // product of the blocks before I for column c of G * K
 #pragma unroll
@@ -552,16 +590,22 @@ __global__ __launch_bounds__(kIntra) void delta_chunk_intra_kernel(DeltaArgs a) 
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int t = 16 * I + 4 * g + j;
-                if (isv) uv[t * P + c] = X[I][j];
-                else wk[t * N + c] = X[I][j];
+                if (isv) uv[(tile * kDCh + t) * 16 + r] = X[I][j];
+                else Q[t * SN + c] = X[I][j];          // q is not needed any more
             }
         }
+    }
+    __syncthreads();
+    float4* wk = reinterpret_cast<float4*>(a.wk + unit * (kDCh * N));
+    for (int i = tid; i < 16 * N; i += kIntra) {
+        const int rr = i & 15, gg = (i >> 4) & 3, tl = i >> 6, blk = tl / nt;
+        wk[i] = *reinterpret_cast<const float4*>(Q + (16 * blk + rr) * SN + 16 * (tl - blk * nt) + 4 * gg);
     }
 }
 
 // One workgroup per (head, 16 state columns, row).  Wave w forms U for the tokens 16 w .. + 15 of a chunk and owns the
-// state rows of the 16-row tiles w, w + 4, ...; the state (as operand) and U pass through LDS.  NT: 16-row tiles.
-template <int NT>
+// state rows of the 16-row tiles w, w + 4, ...; the state (as operand) and U pass through LDS.  NT: 16-row tiles; FULL: the state has exactly NT of them (no tests between the products).
+template <int NT, bool FULL>
 __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
     constexpr int OWN = (NT + 3) / 4;
     __shared__ float Ss[NT * 16][20];
@@ -590,64 +634,60 @@ __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
         f32x4_t uv;
     };
     auto fetch = [&](int64_t unit, Operands& x) {
-        const float* w = a.wk + unit * (kDCh * N) + (16 * wv + r) * N + 4 * g;
+        const float4* w = reinterpret_cast<const float4*>(a.wk + unit * (kDCh * N)) + wv * nt * 64 + lane;
 #pragma unroll
         for (int i = 0; i < NT; ++i)
-            if (i < nt) x.wk[i] = *reinterpret_cast<const float4*>(w + 16 * i);
+            if (FULL || i < nt) x.wk[i] = w[64 * i];
 #pragma unroll
         for (int o = 0; o < OWN; ++o) {
             const int it = wv + 4 * o;
-            if (it < nt) {
-                const float* k = a.kt + unit * (kDCh * N) + (16 * it + r) * kDCh + 4 * g;
+            if (it < nt || (FULL && NT % 4 == 0)) {
+                const float4* k = reinterpret_cast<const float4*>(a.kt + unit * (kDCh * N)) + it * 256 + lane;
 #pragma unroll
-                for (int t = 0; t < 4; ++t) x.kt[o][t] = *reinterpret_cast<const float4*>(k + 16 * t);
+                for (int t = 0; t < 4; ++t) x.kt[o][t] = k[64 * t];
                 x.gm[o] = *reinterpret_cast<const float4*>(a.gc + unit * N + 16 * it + 4 * g);
             }
         }
-        const float* up = a.uv + unit * (kDCh * P) + (16 * wv + 4 * g) * P + c0 + r;
+        const float* up = a.uv + unit * (kDCh * P) + (c0 / 16) * (kDCh * 16) + (16 * wv + 4 * g) * 16 + r;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) x.uv[j] = up[j * P];
+        for (int j = 0; j < 4; ++j) x.uv[j] = up[j * 16];
     };
-    Operands cur, nxt;
-    fetch(u0, cur);
-    nxt = cur;
-    __syncthreads();
-    for (int c = 0; c < nch; ++c) {
+    // three sets of operands: a chunk's are requested while the two before it are worked on
+    auto body = [&](Operands& cur, int c) {
         const int64_t unit = u0 + (int64_t)c * a.H;
-        if (c + 1 < nch) fetch(unit + a.H, nxt);     // under way while this chunk is worked on
         // two accumulators: neighbouring products do not wait for each other
-        f32x4_t x0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, x1 = x0;
+        f32x4_t w0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, w1 = w0;
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
-            if (i < nt) {
+            if (FULL || i < nt) {
                 const int k = 16 * i + 4 * g;
-                MV_DMFMA(x0, cur.wk[i].x, Ss[k][r]);
-                MV_DMFMA(x1, cur.wk[i].y, Ss[k + 1][r]);
-                MV_DMFMA(x0, cur.wk[i].z, Ss[k + 2][r]);
-                MV_DMFMA(x1, cur.wk[i].w, Ss[k + 3][r]);
+                MV_DMFMA(w0, cur.wk[i].x, Ss[k][r]);
+                MV_DMFMA(w1, cur.wk[i].y, Ss[k + 1][r]);
+                MV_DMFMA(w0, cur.wk[i].z, Ss[k + 2][r]);
+                MV_DMFMA(w1, cur.wk[i].w, Ss[k + 3][r]);
             }
         }
-        float* up = a.uv + unit * (kDCh * P) + (16 * wv + 4 * g) * P + c0 + r;
+        float* up = a.uv + unit * (kDCh * P) + (c0 / 16) * (kDCh * 16) + (16 * wv + 4 * g) * 16 + r;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const float u = cur.uv[j] - (x0[j] + x1[j]);
+            const float u = cur.uv[j] - (w0[j] + w1[j]);
             Us[16 * wv + 4 * g + j][r] = u;
-            up[j * P] = u;
+            up[j * 16] = u;
         }
-        float* sp = a.s0 + unit * ((int64_t)N * P) + c0 + r;
+        float* sp = a.s0 + unit * ((int64_t)N * P) + (c0 / 16) * (N * 16) + r;
 #pragma unroll
         for (int o = 0; o < OWN; ++o) {
             const int it = wv + 4 * o;
-            if (it < nt) {
+            if (it < nt || (FULL && NT % 4 == 0)) {
 #pragma unroll
-                for (int j = 0; j < 4; ++j) sp[(int64_t)(16 * it + 4 * g + j) * P] = S[o][j];    // what this chunk starts from
+                for (int j = 0; j < 4; ++j) sp[(16 * it + 4 * g + j) * 16] = S[o][j];    // what this chunk starts from
             }
         }
         __syncthreads();
 #pragma unroll
         for (int o = 0; o < OWN; ++o) {
             const int it = wv + 4 * o;
-            if (it >= nt) continue;
+            if (it >= nt && !(FULL && NT % 4 == 0)) continue;
             f32x4_t y0 = f32x4_t{S[o][0] * cur.gm[o].x, S[o][1] * cur.gm[o].y, S[o][2] * cur.gm[o].z, S[o][3] * cur.gm[o].w};
             f32x4_t y1 = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -664,8 +704,18 @@ __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
                 Ss[16 * it + 4 * g + j][r] = S[o][j];
             }
         }
+        if (c + 3 < nch) fetch(unit + 3 * (int64_t)a.H, cur);
         __syncthreads();
-        cur = nxt;
+    };
+    Operands x0, x1, x2;
+    fetch(u0, x0);
+    if (nch > 1) fetch(u0 + a.H, x1);
+    if (nch > 2) fetch(u0 + 2 * (int64_t)a.H, x2);
+    __syncthreads();
+    for (int c = 0; c < nch; c += 3) {
+        body(x0, c);
+        if (c + 1 < nch) body(x1, c + 1);
+        if (c + 2 < nch) body(x2, c + 2);
     }
 #pragma unroll
     for (int o = 0; o < OWN; ++o)
@@ -677,7 +727,15 @@ __global__ __launch_bounds__(256) void delta_chunk_carry_kernel(DeltaArgs a) {
 }
 
 // One workgroup per (head, chunk), 16 tokens a wave: lane (r, g) ends with token r, columns 16 ct + 4 g .. + 3.
-template <bool F32, int PT>
+// FULL: exactly PT tiles of 16 columns (no tests between the products).
+template <int PT, bool FULL>
+__device__ __forceinline__ void load_slabs(f32x4_t (&x)[PT], const float* src, int64_t slab, int pt) {
+#pragma unroll
+    for (int ct = 0; ct < PT; ++ct)
+        if (FULL || ct < pt) x[ct] = *reinterpret_cast<const f32x4_t*>(src + ct * slab);
+}
+
+template <bool F32, int PT, bool FULL>
 __global__ __launch_bounds__(256) void delta_chunk_inter_kernel(DeltaArgs a) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int h = blockIdx.x, ch = blockIdx.y, tid = threadIdx.x;
@@ -688,43 +746,57 @@ __global__ __launch_bounds__(256) void delta_chunk_inter_kernel(DeltaArgs a) {
     f32x4_t o[PT];
 #pragma unroll
     for (int ct = 0; ct < PT; ++ct) o[ct] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    const float* qd = a.qd + unit * (kDCh * N) + (16 * wv + r) * N + 4 * g;
+    const float4* qd = reinterpret_cast<const float4*>(a.qd + unit * (kDCh * N)) + wv * (N / 16) * 64 + lane;
     const float* bm = a.bm + unit * (kDCh * kDCh) + (16 * wv + r) * kDCh + 4 * g;
     const float* s0 = a.s0 + unit * ((int64_t)N * P);
     const float* uv = a.uv + unit * (kDCh * P);
-    const int P4 = P / 4;
-    // 64 rows of the right-hand operand at a time: the state's, then U's
-    for (int k0 = 0; k0 < N + kDCh; k0 += kDCh) {
-        const bool isu = k0 >= N;
-        const int rows = isu ? kDCh : (N - k0 < kDCh ? N - k0 : kDCh);
-        const float* src = isu ? uv : s0 + (int64_t)k0 * P;
-        __syncthreads();
-        for (int i = tid; i < rows * P4; i += 256) {
-            const int rr = i / P4, cc = i - rr * P4;
-            *reinterpret_cast<float4*>(lds + rr * SP + 4 * cc) = *reinterpret_cast<const float4*>(src + (int64_t)rr * P + 4 * cc);
-        }
-        __syncthreads();
-        const int top = isu ? 16 * (wv + 1) : rows;      // tokens behind the wave's own do not enter
-        for (int k = 0; k < top; k += 16) {
-            const float4 w = *reinterpret_cast<const float4*>(isu ? bm + k : qd + k0 + k);
-            const float* s = lds + (k + 4 * g) * SP + r;
+    // 64 rows of the right-hand operand at a time - the state's, then U's - through LDS, the next ones in registers
+    // while these are used.  Slabs of 16 columns: thread (tid / 4, tid % 4) moves one 16-byte piece of a row per slab.
+    const int stages = (N + kDCh - 1) / kDCh + 1, sr = tid >> 2, sc = 4 * (tid & 3);
+    f32x4_t nx[PT], nw[4];        // the next stage's rows, and the wave's left-hand operand for them
+    const int nt = N / 16;
 #pragma unroll
-            for (int ct = 0; ct < PT; ++ct) {
-                if (ct < pt) {
-                    MV_DMFMA(o[ct], s[16 * ct], w.x);
-                    MV_DMFMA(o[ct], s[SP + 16 * ct], w.y);
-                    MV_DMFMA(o[ct], s[2 * SP + 16 * ct], w.z);
-                    MV_DMFMA(o[ct], s[3 * SP + 16 * ct], w.w);
-                }
+    for (int k = 0; k < 4; ++k) nw[k] = *reinterpret_cast<const f32x4_t*>(qd + (k < nt ? k : nt - 1) * 64);
+    load_slabs<PT, FULL>(nx, s0 + (sr < N ? sr : N - 1) * 16 + sc, (int64_t)N * 16, pt);
+    for (int stage = 0; stage < stages; ++stage) {
+        const bool isu = stage == stages - 1;
+        const int k0 = stage * kDCh;
+        __syncthreads();
+#pragma unroll
+        for (int ct = 0; ct < PT; ++ct)
+            if (FULL || ct < pt) *reinterpret_cast<f32x4_t*>(lds + sr * SP + 16 * ct + sc) = nx[ct];
+        f32x4_t w[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) w[k] = nw[k];
+        __syncthreads();
+        if (!isu) {
+            const bool nu = stage + 1 == stages - 1;
+            const int n0 = k0 + kDCh, rows = nu ? kDCh : N - n0;
+            load_slabs<PT, FULL>(nx, (nu ? uv : s0 + n0 * 16) + (sr < rows ? sr : rows - 1) * 16 + sc, (int64_t)(nu ? kDCh : N) * 16, pt);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const int i = n0 / 16 + k;
+                nw[k] = nu ? *reinterpret_cast<const f32x4_t*>(bm + 16 * k) : *reinterpret_cast<const f32x4_t*>(qd + (i < nt ? i : nt - 1) * 64);
             }
         }
-        if (isu) break;
-        if (k0 + kDCh >= N) k0 = N - kDCh;               // U's rows come next, whatever N is
+        // of the state what is left, of U no tokens behind the wave's own
+        const int top = isu ? 16 * (wv + 1) : (N - k0 < kDCh ? N - k0 : kDCh);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            if (16 * k >= top) break;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const float* s = lds + (16 * k + 4 * g + j) * SP + r;
+#pragma unroll
+                for (int ct = 0; ct < PT; ++ct)
+                    if (FULL || ct < pt) MV_DMFMA(o[ct], s[16 * ct], w[k][j]);
+            }
+        }
     }
     float ss = 0.f;
 #pragma unroll
     for (int ct = 0; ct < PT; ++ct)
-        if (ct < pt) ss += o[ct][0] * o[ct][0] + o[ct][1] * o[ct][1] + o[ct][2] * o[ct][2] + o[ct][3] * o[ct][3];
+        if (FULL || ct < pt) ss += o[ct][0] * o[ct][0] + o[ct][1] * o[ct][1] + o[ct][2] * o[ct][2] + o[ct][3] * o[ct][3];
     ss += __shfl_xor(ss, 16, 64);
     ss += __shfl_xor(ss, 32, 64);
     const int t = 16 * wv + r;
@@ -734,7 +806,16 @@ __global__ __launch_bounds__(256) void delta_chunk_inter_kernel(DeltaArgs a) {
     typename ActD<F32>::T* op = (typename ActD<F32>::T*)a.out + (int64_t)(start + t) * a.ldo + (int64_t)h * p;
 #pragma unroll
     for (int ct = 0; ct < PT; ++ct) {
-        if (ct >= pt) continue;
+        if (!FULL && ct >= pt) continue;
+        if (a.vec) {        // p a multiple of 16, rows aligned for four values at a time
+            const int c = 16 * ct + 4 * g;
+            const float4 z = *reinterpret_cast<const float4*>(zp + c), w = *reinterpret_cast<const float4*>(a.norm + c);
+            const float4 y = make_float4((o[ct][0] * inv) * w.x * sigmoid_d(z.x), (o[ct][1] * inv) * w.y * sigmoid_d(z.y),
+                                         (o[ct][2] * inv) * w.z * sigmoid_d(z.z), (o[ct][3] * inv) * w.w * sigmoid_d(z.w));
+            if (F32) *reinterpret_cast<float4*>((float*)op + c) = y;
+            else *reinterpret_cast<uint2*>((uint16_t*)op + c) = make_uint2(pack_bf16x2(y.x, y.y), pack_bf16x2(y.z, y.w));
+            continue;
+        }
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int c = 16 * ct + 4 * g + j;
@@ -838,6 +919,7 @@ int mv_delta_rule(const float* qkv, int64_t ldq, const float* gate_in, int64_t l
     a.r = DeltaRows{nullptr, row_start, row_len, row_ctx, row_slot};
     a.K = kv_heads; a.H = heads; a.n = n; a.p = p; a.max_len = chunks > 0 ? max_len : 0; a.eps = eps;
     a.ch_start = ch_start; a.ch_len = ch_len; a.row_ch0 = row_ch0; a.row_nch = row_nch;
+    a.vec = p % 16 == 0 && ldz % 4 == 0 && ldo % 4 == 0 && aligned16(z) && aligned16(out) && aligned16(norm);
     hipStream_t s = (hipStream_t)stream;
     if (chunks == 0 || short_tokens != 0) {
         int pw = 16;
@@ -870,27 +952,35 @@ int mv_delta_rule(const float* qkv, int64_t ldq, const float* gate_in, int64_t l
         a.s0 = a.bm + U * kDCh * kDCh;
         a.gc = a.s0 + U * N * P;
         const size_t lds1 = delta_intra_lds(n), lds2 = (size_t)kDCh * (P + 4) * sizeof(float);
-        static LdsOptIn o1, o2[2][4];
+        static LdsOptIn o1, o2[2][6];
         if (int rc = ensure_dynamic_lds((const void*)delta_chunk_intra_kernel, lds1, o1)) return rc;
         hipLaunchKernelGGL(delta_chunk_intra_kernel, dim3(heads, chunks), dim3(kIntra), lds1, s, a);
         const dim3 gc(heads, (unsigned)(P / 16), rows);
-        if (N <= 32) hipLaunchKernelGGL(delta_chunk_carry_kernel<2>, gc, dim3(256), 0, s, a);
-        else if (N <= 64) hipLaunchKernelGGL(delta_chunk_carry_kernel<4>, gc, dim3(256), 0, s, a);
-        else if (N <= 128) hipLaunchKernelGGL(delta_chunk_carry_kernel<8>, gc, dim3(256), 0, s, a);
-        else hipLaunchKernelGGL(delta_chunk_carry_kernel<10>, gc, dim3(256), 0, s, a);
+        if (N == 128) hipLaunchKernelGGL((delta_chunk_carry_kernel<8, true>), gc, dim3(256), 0, s, a);
+        else if (N == 64) hipLaunchKernelGGL((delta_chunk_carry_kernel<4, true>), gc, dim3(256), 0, s, a);
+        else if (N <= 32) hipLaunchKernelGGL((delta_chunk_carry_kernel<2, false>), gc, dim3(256), 0, s, a);
+        else if (N <= 64) hipLaunchKernelGGL((delta_chunk_carry_kernel<4, false>), gc, dim3(256), 0, s, a);
+        else if (N <= 128) hipLaunchKernelGGL((delta_chunk_carry_kernel<8, false>), gc, dim3(256), 0, s, a);
+        else hipLaunchKernelGGL((delta_chunk_carry_kernel<10, false>), gc, dim3(256), 0, s, a);
         const dim3 gi(heads, chunks);
-#define MV_DELTA_INTER(F32_, PT_, IDX_)                                                                                    \
+#define MV_DELTA_INTER(F32_, PT_, FULL_, IDX_)                                                                             \
     do {                                                                                                               \
-        if (int rc = ensure_dynamic_lds((const void*)delta_chunk_inter_kernel<F32_, PT_>, lds2, o2[F32_][IDX_])) return rc;  \
-        hipLaunchKernelGGL((delta_chunk_inter_kernel<F32_, PT_>), gi, dim3(256), lds2, s, a);                             \
+        const void* fn = (const void*)delta_chunk_inter_kernel<F32_, PT_, FULL_>;                                          \
+        if (int rc = ensure_dynamic_lds(fn, lds2, o2[F32_][IDX_])) return rc;                                             \
+        hipLaunchKernelGGL((delta_chunk_inter_kernel<F32_, PT_, FULL_>), gi, dim3(256), lds2, s, a);                       \
     } while (0)
-        if (f32) {
-            if (P <= 32) MV_DELTA_INTER(true, 2, 0); else if (P <= 64) MV_DELTA_INTER(true, 4, 1);
-            else if (P <= 128) MV_DELTA_INTER(true, 8, 2); else MV_DELTA_INTER(true, 16, 3);
-        } else {
-            if (P <= 32) MV_DELTA_INTER(false, 2, 0); else if (P <= 64) MV_DELTA_INTER(false, 4, 1);
-            else if (P <= 128) MV_DELTA_INTER(false, 8, 2); else MV_DELTA_INTER(false, 16, 3);
-        }
+#define MV_DELTA_INTER_P(F32_)                                                                                         \
+    do {                                                                                                               \
+        if (P == 128) MV_DELTA_INTER(F32_, 8, true, 0);                                                                  \
+        else if (P == 64) MV_DELTA_INTER(F32_, 4, true, 1);                                                              \
+        else if (P <= 32) MV_DELTA_INTER(F32_, 2, false, 2);                                                             \
+        else if (P <= 64) MV_DELTA_INTER(F32_, 4, false, 3);                                                             \
+        else if (P <= 128) MV_DELTA_INTER(F32_, 8, false, 4);                                                            \
+        else MV_DELTA_INTER(F32_, 16, false, 5);                                                                         \
+    } while (0)
+        if (f32) MV_DELTA_INTER_P(true);
+        else MV_DELTA_INTER_P(false);
+#undef MV_DELTA_INTER_P
 #undef MV_DELTA_INTER
     }
     return check_launch();
