@@ -574,10 +574,11 @@ int mv_qk_rotary_store(float* qk, int64_t ld, const float* q_bias, const float* 
  * is read once for those heads - and, with splits > 1, a second launch merges the splits' pieces.
  * short_tokens: how many of the step's tokens lie in rows of up to max_len tokens (-1: not known); 0 lets a step whose
  * rows all went to the tiled kernel skip the launch of the per-token form.  gate != NULL (fp32 [tokens, heads * dv]):
- * out is multiplied by sigmoid(gate) before it is rounded.  With a chunk table (chunks > 0:
+ * out is multiplied by sigmoid(gate) before it is rounded.  chunked != 0: a token sees its own chunk of `window` positions
+ * (counted from position 0) up to itself instead of the last `window` positions.  With a chunk table (chunks > 0:
  * rows of more than max_len tokens cut into runs of up to 64, as for mv_scan_chunked; row_len per row), bf16
  * and a head shape the tiled kernel is built for - (d, dv) in (32,32) (64,64) (96,96) (128,128) (128,64)
- * (64,128), 64-token pages - those rows run on the matrix cores, a workgroup per (chunk, head): q.k in bf16
+ * (64,128) (64,32), 64-token pages - those rows run on the matrix cores, a workgroup per (chunk, head): q.k in bf16
  * (q rounded as the cached keys are), softmax in fp32, P.V with fp32 P.  Every other token takes the
  * one-workgroup-per-(token, head) form. */
 int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void* v_cache, void* out, int64_t ldo,
@@ -585,7 +586,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
                    int page, const float* slopes, int tokens, int heads, int kv_heads, int d, int dv, float scale,
                    int window, int f32, const int32_t* row_len, const int32_t* ch_start, const int32_t* ch_len,
                    int chunks, int max_len, int keep_first, const float* sinks, float* part, int splits,
-                   int short_tokens, const float* gate, int64_t ldg, mv_stream_t stream);
+                   int short_tokens, const float* gate, int64_t ldg, int chunked, mv_stream_t stream);
 /* How many splits of the keys mv_window_attn should be given for a step of `tokens` tokens (1: none). */
 int mv_window_attn_splits(int tokens, int heads, int kv_heads, int window, int keep_first);
 
@@ -716,6 +717,12 @@ int mv_moe_combine(const float* expert_out, int64_t lde, const int32_t* place, c
  * renormalised. */
 int mv_moe_route_sigmoid(const void* h, int64_t ldh, const float* w_router, int32_t* ids, float* weights, int tokens,
                          int n, int experts, int top, int f32, mv_stream_t stream);
+/* scores = sigmoid(fp32 logits); the experts form `groups` equal runs of neighbours, each worth the sum of its two largest
+ * score + correction (correction == NULL: none); the `top` largest score + correction within the `keep` best runs are
+ * chosen (ties: the lower index; top <= keep * experts / groups), weights = their scores, not renormalised. */
+int mv_moe_route_grouped(const void* h, int64_t ldh, const float* w_router, const float* correction, int32_t* ids,
+                         float* weights, int tokens, int n, int experts, int groups, int keep, int top, int f32,
+                         mv_stream_t stream);
 /* mv_gated_act on rows sorted by expert, with both halves scaled first: out = act( f(s a[:, :n]) * (s a[:, n:2n]) ),
  * s = scale[order[row]] (order == NULL: scale[row]): an expert that reads weight * h, from the products of h. */
 int mv_gated_act_scaled(const float* a, int64_t lda, void* out, int64_t ldo, int rows, int n, int kind, float limit,
@@ -807,6 +814,48 @@ int mv_delta_rule(const float* qkv, int64_t ldq, const float* gate_in, int64_t l
                   int chunks, int max_len, int short_tokens, int f32, mv_stream_t stream);
 int mv_delta_chunked_ok(int n, int p);
 int64_t mv_delta_scratch_floats(int n, int p);
+
+/* ---- per-head norms with rotation, gated linear attention, layer norm on outputs (seq_mix.hip, gla.hip, stream_ops.hip) ---- */
+
+/* qkv [T, ld] = q [heads * d] | k [kv_heads * d] | v [kv_heads * dv] of one projection.  Every head of q and of k gets its
+ * bias, an RMS norm over itself (q_norm / k_norm [d], shared by the heads; NULL: no norm) and the rotation of its first
+ * `rot` dimensions (angle = position * inv_freq; `adjacent` pairs, or halves); q stays in place, k goes to its page; v
+ * gets its bias and goes to its page.  low_out [T, low_n] (low_n > 0) = the columns low [T, ldl] in the activation type.
+ * d - rot / 2 <= 512. */
+int mv_qkv_headnorm_rotary_store(float* qkv, int64_t ld, const float* q_bias, const float* k_bias, const float* v_bias,
+                                 const float* q_norm, const float* k_norm, float eps, const double* inv_freq,
+                                 void* k_cache, void* v_cache, const int32_t* tok_row, const int32_t* tok_pos,
+                                 const int32_t* block_table, int bt_stride, int page, int tokens, int heads,
+                                 int kv_heads, int d, int dv, int rot, int adjacent, const float* low, int64_t ldl,
+                                 void* low_out, int low_n, int f32, mv_stream_t stream);
+
+/* Per head, S [n, p] kept in state[slot] (zero where row_ctx == 0): S = diag(sigmoid(z + z_bias)^inv_tau) S + k v^T,
+ * o = S^T (q * q_scale), out = act( o / sqrt(mean(o^2) + eps) * norm[p] * gate * sigmoid(gate) ).  q, k, z [T, heads * n],
+ * v, gate [T, heads * p], z_bias [heads * n] or NULL.  Rows of up to max_len tokens (every row when chunks == 0) run token
+ * by token (p <= 256, n times p rounded up to a power of two <= 65536), longer ones in chunks of 64 where
+ * mv_gated_linear_chunked_ok(n, p) (n, p <= 256); scratch: chunks * heads * mv_gated_linear_scratch_floats(n, p) floats,
+ * 16-byte aligned.  short_tokens: tokens in rows outside the chunk table (0: none, -1: unknown). */
+int mv_gated_linear_attn(const float* q, int64_t ldq, const float* k, int64_t ldk, const float* v, int64_t ldv,
+                         const float* z, int64_t ldz, const float* z_bias, const float* gate, int64_t ldg,
+                         const float* norm, float* state, void* out, int64_t ldo, const int32_t* row_start,
+                         const int32_t* row_len, const int32_t* row_ctx, const int32_t* row_slot, int rows, int heads,
+                         int n, int p, float q_scale, float inv_tau, float eps, float* scratch, const int32_t* ch_start,
+                         const int32_t* ch_len, const int32_t* row_ch0, const int32_t* row_nch, int chunks, int max_len,
+                         int short_tokens, int f32, mv_stream_t stream);
+int mv_gated_linear_chunked_ok(int n, int p);
+int64_t mv_gated_linear_scratch_floats(int n, int p);
+
+/* x += LN(v), LN(v) = (v - mean(v)) / sqrt(mean((v - mean)^2) + eps) * w; h (NULL: none) = act(x), or with next_w act of that
+ * layer norm of the new x.  v = y1; or with y2 (and r1, r2) s * (rms(y1) * r1 + rms(y2) * r2), rms(y) = y / sqrt(mean(y^2) +
+ * eps); or with `place` [rows, top] the sum of weights[r, k] * y1[place[r, k], :] (+ y2[r, :]).  n <= 16384 where every row is
+ * 16-byte aligned. */
+int mv_layernorm_residual(const float* y1, int64_t ld1, const float* r1, const float* y2, int64_t ld2, const float* r2,
+                          float s, const int32_t* place, const float* weights, int top, const float* w, float eps,
+                          const float* next_w, float* x, int64_t ldx, void* h, int64_t ldh, int rows, int n, int f32,
+                          mv_stream_t stream);
+/* out[r,:] = act( LN(x[idx[r],:]) ); idx == NULL: row r itself. */
+int mv_layernorm_gather(const float* x, int64_t ldx, const int32_t* idx, const float* w, float eps, void* out,
+                        int64_t ldo, int rows, int n, int f32, mv_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -108,7 +108,7 @@ PROTOTYPES = {
     "mv_gated_group_norm": (_I, [_P, _L, _P, _L, _P, _P, _L, _I, _I, _I, _I, _I, _F, _I, _P]),
     "mv_qk_unitnorm_store": (_I, [_P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P]),
     "mv_window_attn": (_I, [_P, _L, _P, _P, _P, _L, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _F, _I, _I,
-                            _P, _P, _P, _I, _I, _I, _P, _P, _I, _I, _P, _L, _P]),
+                            _P, _P, _P, _I, _I, _I, _P, _P, _I, _I, _P, _L, _I, _P]),
     "mv_window_attn_splits": (_I, [_I, _I, _I, _I, _I]),
     "mv_qk_rotary_store": (_I, [_P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _L, _P, _L,
                                 _I, _I, _F, _F, _I, _P]),
@@ -157,6 +157,15 @@ PROTOTYPES = {
                            _P, _P, _P, _P, _I, _I, _I, _I, _P]),
     "mv_delta_chunked_ok": (_I, [_I, _I]),
     "mv_delta_scratch_floats": (_L, [_I, _I]),
+    "mv_moe_route_grouped": (_I, [_P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "mv_qkv_headnorm_rotary_store": (_I, [_P, _L, _P, _P, _P, _P, _P, _F, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I,
+                                          _I, _I, _P, _L, _P, _I, _I, _P]),
+    "mv_gated_linear_attn": (_I, [_P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _L, _P, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I,
+                                  _F, _F, _F, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P]),
+    "mv_gated_linear_chunked_ok": (_I, [_I, _I]),
+    "mv_gated_linear_scratch_floats": (_L, [_I, _I]),
+    "mv_layernorm_residual": (_I, [_P, _L, _P, _P, _L, _P, _F, _P, _P, _I, _P, _F, _P, _P, _L, _P, _L, _I, _I, _I, _P]),
+    "mv_layernorm_gather": (_I, [_P, _L, _P, _P, _F, _P, _L, _I, _I, _I, _P]),
     "mv_graph_begin_capture": (_I, [_P]),
     "mv_graph_end_capture": (_I, [_P, ctypes.POINTER(c_void_p)]),
     "mv_graph_launch": (_I, [_P, _P]),

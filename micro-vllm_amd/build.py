@@ -33,6 +33,7 @@ SOURCES = [
     "moe.hip",
     "diff_attn.hip",
     "delta.hip",
+    "gla.hip",
 ]
 
 # Libraries that hold a part of the sources, `lib/libmvllm_<name>.so`: what one model family needs, for a
@@ -42,7 +43,7 @@ SETS = {
     # fp32 residual stream, recurrent mixers, windowed attention; the wave-tile projections for the
     # shapes they take, and the sampler
     "ragged": ["runtime.hip", "linear_any.hip", "stream_ops.hip", "seq_mix.hip", "latent_attn.hip", "moe.hip",
-               "diff_attn.hip", "delta.hip", "elementwise.hip", "wgemm.hip", "gemm_prefill.hip", "sampler.hip"],
+               "diff_attn.hip", "delta.hip", "gla.hip", "elementwise.hip", "wgemm.hip", "gemm_prefill.hip", "sampler.hip"],
 }
 
 # -ffp-contract=off: rounding is part of the parity contract; FMAs are written explicitly

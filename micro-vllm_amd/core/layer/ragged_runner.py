@@ -77,6 +77,17 @@ Per layer (Dugazen; an RMS norm with weight 1 + w in front of every sublayer and
             with the first mixing layer's, keys and values into the pages, in one launch -> windowed softmax attention
             with the sigmoid gate on its output -> out-projection
   dense     gate|up projection -> clamped gate -> down
+
+Per layer (Sizizen; a layer norm on every sublayer's output, none in front of it):
+  parallel  ONE projection gives both mixers' q | k | v, the right one's gate and its low-rank columns
+            left: biases, norm per head of q and k, rotation, keys and values into the pages, the low-rank columns cast,
+            in one launch -> softmax attention within chunks of positions -> out-projection
+            right: low-rank columns to decay logits -> decays, gated linear attention (state per slot), unit-RMS per head,
+            weight, SiLU gate, in one call -> out-projection
+  residual  x += LN of half the sum of both outputs, each normed over the width first, in one launch
+  dense     gate|up projection -> SiLU gate -> down -> x += LN of it
+  moe       router (fp32, sigmoid scores, group-limited choice) -> pairs sorted by expert -> up by segment -> squared
+            ReLU -> down by segment; shared expert beside it; x += LN of the weighted sum, in one launch
 """
 import logging
 import math
@@ -85,7 +96,7 @@ from typing import Dict, List, Optional
 import torch
 
 from ...kernel import ragged_ops as ops
-from ...models import dugazen
+from ...models import dugazen, sizizen
 from ...models.nesisun import GATE_SLOPE, WEIGHT_SUM_FLOOR
 from ...models.pagazen import mamba2_sizes
 from ..state_cache import HybridCacheManager, RaggedStep
@@ -122,6 +133,7 @@ class RaggedRunner:
         self.parallel_prenorm = cfg.architecture == "Nesisun"   # one RMS norm feeds mixer and feed-forward alike
         self.gated_prenorm = cfg.architecture == "Solopel"      # pre-norm layers whose sublayer outputs pass a gate
         self.double_norm = cfg.architecture == "Dugazen"        # an RMS norm in front of every sublayer and one behind it
+        self.post_layernorm = cfg.architecture == "Sizizen"     # a layer norm behind every sublayer, none in front
         for wi, layer in self.runs:
             if wi not in self._w:
                 self._w[wi] = self._prepare_layer(wi, layer)
@@ -181,6 +193,8 @@ class RaggedRunner:
             return self._prepare_solopel(i, layer)
         if self.double_norm:
             return self._prepare_dugazen(i, layer)
+        if self.post_layernorm:
+            return self._prepare_sizizen(i, layer)
         g, p, m = self.model.get, f"l{i}.", layer["mixer"]
         w = {"norm1": self._small(g(p + "norm1"))}
         if layer["type"] == "mamba2":
@@ -354,6 +368,45 @@ class RaggedRunner:
                      gate_up=self._linear(g(p + "mlp.gate"), g(p + "mlp.up")), down=self._linear(g(p + "mlp.down")))
         return w
 
+    def _prepare_sizizen(self, i: int, layer: dict) -> dict:
+        g, p, m, W = self.model.get, f"l{i}.", layer["mixer"], self.width
+        L, R = m["left"], m["right"]
+        left, right = p + "mix.left.", p + "mix.right."
+        rot = int(L["rot"]["dims"])
+        inv_freq = float(L["rot"]["base"]) ** (-2.0 * torch.arange(max(rot // 2, 1), dtype=torch.float64) / max(rot, 1))
+        a1, a2 = g(right + "a1"), g(right + "a2")
+        rank = a1.shape[0]
+        low = -(-rank // 64) * 64               # an inner width the wave-tile projections take
+        C = (int(L["heads"]) + int(L["kv_heads"])) * int(L["dim"]) + int(L["kv_heads"]) * int(L["vdim"])
+        D = int(R["heads"]) * 2 * (int(R["dim"]) + int(R["vdim"]))
+        rows = lambda n: torch.zeros(n, W, dtype=a1.dtype)   # noqa: E731
+        # [left q | k | v (| zeros) | right q | k | v | g (| zeros) | a1 (| zeros)]: every section starts at a multiple of 16
+        off = C + (-C % 16)
+        low_off = off + D + (-D % 16)
+        second = torch.zeros(a2.shape[0], low, dtype=a2.dtype)
+        second[:, :rank] = a2
+        w = {"norm1": self._small(g(p + "norm1")), "right_off": off, "low_off": low_off, "low": low,
+             "w_in": self._linear(g(left + "q"), g(left + "k"), g(left + "v"), rows(off - C), g(right + "q"), g(right + "k"),
+                                  g(right + "v"), g(right + "g"), rows(low_off - off - D), a1, rows(low - rank)),
+             "w_second": self._linear(second), "left_o": self._linear(g(left + "o")), "right_o": self._linear(g(right + "o")),
+             "inv_freq": inv_freq.to(self.device)}
+        w.update({k: self._small(g(p + "mix." + n)) for k, n in (
+            ("q_b", "left.q.b"), ("k_b", "left.k.b"), ("v_b", "left.v.b"), ("q_norm", "left.q.norm"), ("k_norm", "left.k.norm"),
+            ("left_out", "left.out"), ("right_out", "right.out"), ("norm", "right.norm"), ("z_b", "right.a2.b"))})
+        mlp = layer.get("mlp")
+        if mlp:
+            w["norm2"] = self._small(g(p + "norm2"))
+            if mlp["kind"] == "dense":
+                w.update(gate_up=self._linear(g(p + "mlp.gate"), g(p + "mlp.up")), down=self._linear(g(p + "mlp.down")))
+            else:
+                E = int(mlp["router"]["experts"])
+                w.update(router=self._small(g(p + "mlp.router")), correction=self._small(g(p + "mlp.correction")),
+                         e_up=self._stacked([g(p + f"mlp.e{e}.up") for e in range(E)]),
+                         e_down=self._stacked([g(p + f"mlp.e{e}.down") for e in range(E)]))
+                if mlp.get("shared"):
+                    w.update(s_up=self._linear(g(p + "mlp.shared.up")), s_down=self._linear(g(p + "mlp.shared.down")))
+        return w
+
     # ------------------------------------------------------------------ cache geometry
     def cache_layout(self):
         """(kv_layers, state_layers) for HybridCacheManager: what every layer RUN keeps per sequence."""
@@ -391,7 +444,7 @@ class RaggedRunner:
             elif layer["type"] in ("latent_attention", "latent_attention_2"):
                 kv[i] = (1, int(m["kv_rank"]) + int(m["rot_dim"]), 0)    # one latent + rotated key part per token
                 state[i] = {"shift": (self.width,)}
-            else:
+            else:      # two mixers side by side: pages for the left one, a memory per head for the right one
                 L, R = m["left"], m["right"]
                 kv[i] = (int(L["kv_heads"]), int(L["dim"]), int(L["vdim"]))
                 state[i] = {"ret": (int(R["heads"]), int(R["dim"]), int(R["vdim"]))}
@@ -552,6 +605,10 @@ class RaggedRunner:
             if want is None:
                 normed = self._actbuf(T, self.width)
             self._dugazen_stack(step, cache, residuals, x, h, normed)
+        elif self.post_layernorm:
+            if want is None:
+                normed = self._actbuf(T, self.width)
+            self._sizizen_stack(step, cache, residuals, x, h, normed)
         elif self.sandwich:
             ops.embed_scaled(self.embed, step.ids, 1.0, x, h)
             for li, (wi, layer) in enumerate(self.runs):
@@ -588,6 +645,8 @@ class RaggedRunner:
             ops.dyt_gather(x, want, self.final_norm, normed)
         elif self.parallel_prenorm:
             ops.rmsnorm_gather(x, want, self.final_norm, cfg.eps, normed)
+        elif self.post_layernorm:
+            ops.layernorm_gather(x, want, self.final_norm, cfg.eps, normed)
         else:
             ops.offset_rmsnorm_gather(x, want, self.final_norm, cfg.eps, normed)
         logits = self.head(normed, self._f32buf(rows, self.vocab_size))
@@ -822,6 +881,85 @@ class RaggedRunner:
         ops.window_attn(proj[:, :H * d], kc, vc, a, step, None, H, G, d, dv, float(m["scale"]), window,
                         tiled=self.tiled_attn, part=part, splits=splits, gate=proj[:, C:C + H * dv])
         return w["w_o"](a, self._f32buf(T, self.width))
+
+    # ------------------------------------------------------------------ Sizizen layers
+    def _sizizen_stack(self, step: RaggedStep, cache: HybridCacheManager, residuals, x, h, normed):
+        """All layers on the stream x (fp32, updated in place); h holds the stream in the activation type, which every
+        sublayer reads; `normed` (optional) receives the final norm of the stream."""
+        eps = self.cfg.eps
+        ops.embed_scaled(self.embed, step.ids, 1.0, x, h)
+        for li, (wi, layer) in enumerate(self.runs):
+            w, mlp = self._w[wi], layer.get("mlp")
+            # the last residual step hands out the final norm, or nothing where only some rows of it are wanted
+            last = li + 1 == len(self.runs)
+            end_h, end_w = (normed, self.final_norm if normed is not None else None) if last else (h, None)
+            left, right = self._sizizen_mixers(li, w, layer["mixer"], h, step, cache)
+            branch = (w["left_out"], right, w["right_out"], sizizen.BRANCH_SCALE)
+            if not mlp:
+                ops.layernorm_residual(x, left, w["norm1"], eps, end_h, branch=branch, next_w=end_w)
+            else:
+                ops.layernorm_residual(x, left, w["norm1"], eps, h, branch=branch)
+                if mlp["kind"] == "dense":
+                    ff = int(mlp["ff"])
+                    act = self._actbuf(step.tokens, ff)
+                    ops.gated_act(w["gate_up"](h, self._f32buf(step.tokens, 2 * ff)), act, ops.GATE_SILU)
+                    y = w["down"](act, self._f32buf(step.tokens, self.width))
+                    ops.layernorm_residual(x, y, w["norm2"], eps, end_h, next_w=end_w)
+                else:
+                    down, place, wts, shared = self._grouped_experts(w, mlp, h, step.tokens)
+                    ops.layernorm_residual(x, down, w["norm2"], eps, end_h, place=place, weights=wts, shared=shared,
+                                           next_w=end_w)
+            if residuals is not None:
+                residuals.append(x.clone())
+
+    def _sizizen_mixers(self, li, w, m, h, step: RaggedStep, cache: HybridCacheManager):
+        """Both mixers of a parallel layer on the same input: their outputs (fp32), not yet normed."""
+        T, eps, L, R = step.tokens, self.cfg.eps, m["left"], m["right"]
+        H, G, d, dv = int(L["heads"]), int(L["kv_heads"]), int(L["dim"]), int(L["vdim"])
+        Hr, n, p = int(R["heads"]), int(R["dim"]), int(R["vdim"])
+        proj = w["w_in"](h, self._f32buf(T, w["w_in"].n))      # [q | k | v .. | q | k | v | g .. | low-rank columns ..]
+        kc, vc = cache.k_caches[li], cache.v_caches[li]
+        low = self._actbuf(T, w["low"])
+        ops.qkv_headnorm_rotary_store(proj[:, :(H + G) * d + G * dv], kc, vc, step, H, G, d, dv, w["inv_freq"],
+                                      int(L["rot"]["dims"]), eps, q_bias=w["q_b"], k_bias=w["k_b"], v_bias=w["v_b"],
+                                      q_norm=w["q_norm"], k_norm=w["k_norm"],
+                                      low=proj[:, w["low_off"]:w["low_off"] + w["low"]], low_out=low)
+        a = self._actbuf(T, H * dv)
+        chunk = int(L["mask"]["size"])
+        splits = ops.window_attn_splits(T, H, G, chunk) if self.grouped_attn else 0
+        part = self._f32buf(1, T * H * splits * (dv + 2)) if splits else None
+        ops.window_attn(proj[:, :H * d], kc, vc, a, step, None, H, G, d, dv, float(L["scale"]), chunk,
+                        tiled=self.tiled_attn, part=part, splits=splits, chunked=True)
+        left = w["left_o"](a, self._f32buf(T, self.width))
+
+        z = w["w_second"](low, self._f32buf(T, Hr * n))        # decay logits
+        o = w["right_off"]
+        q, k = proj[:, o:o + Hr * n], proj[:, o + Hr * n:o + 2 * Hr * n]
+        v, g = proj[:, o + 2 * Hr * n:o + 2 * Hr * n + Hr * p], proj[:, o + 2 * Hr * n + Hr * p:o + 2 * Hr * (n + p)]
+        u = self._actbuf(T, Hr * p)
+        ops.gated_linear_attn(q, k, v, z, w["z_b"], g, w["norm"], cache.states[li]["ret"], u, step, Hr, n, p,
+                              float(R["tau"]), eps, q_scale=n ** -0.5, chunked=self.chunked_scan)
+        return left, w["right_o"](u, self._f32buf(T, self.width))
+
+    def _grouped_experts(self, w, mlp, h, T):
+        """Routed squared-ReLU experts: (their outputs sorted by expert, each pair's row there, weights, shared output)."""
+        r = mlp["router"]
+        E, top, ff = int(r["experts"]), int(r["top"]), int(mlp["expert"]["ff"])
+        groups, keep = sizizen.expert_groups(r)
+        ids, wts = self._i32buf(T * top).view(T, top), self._f32buf(T, top)
+        ops.moe_route_grouped(h, w["router"], w["correction"], ids, wts, groups, keep)
+        seg, order, place = self._i32buf(E + 1), self._i32buf(T * top), self._i32buf(T * top)
+        ops.moe_plan(ids, seg, order, place, E)
+        up = ops.linear_segments(h, w["e_up"], self._f32buf(T * top, ff), seg, order, top, T)
+        act = self._actbuf(T * top, ff)
+        ops.relu_squared(up, act)
+        down = ops.linear_segments(act, w["e_down"], self._f32buf(T * top, self.width), seg, None, 1, T)
+        if not mlp.get("shared"):
+            return down, place, wts, None
+        sf = int(mlp["shared"]["ff"])
+        s_act = self._actbuf(T, sf)
+        ops.relu_squared(w["s_up"](h, self._f32buf(T, sf)), s_act)
+        return down, place, wts, w["s_down"](s_act, self._f32buf(T, self.width))
 
     # ------------------------------------------------------------------ Fagunex layers
     def _i32buf(self, count):

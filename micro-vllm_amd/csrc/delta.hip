@@ -9,25 +9,9 @@
 //                  many tokens: chunks of 64 (below).  Both form the gates g = exp(-exp(A) softplus(a + bias)) and
 //                  hand out act( o / rms(o) * w * sigmoid(z) )
 // All of it in fp32; only what goes to a projection is of the activation type.
-#include "common.h"
+#include "recurrence.h"
 
 namespace mv {
-
-template <bool F32> struct ActD;
-template <> struct ActD<true> {
-    typedef float T;
-    static __device__ __forceinline__ void st(float* p, float v) { *p = v; }
-};
-template <> struct ActD<false> {
-    typedef uint16_t T;
-    static __device__ __forceinline__ void st(uint16_t* p, float v) { *p = (uint16_t)f32_to_bf16_bits(v); }
-};
-
-constexpr float kLog2E = 1.4426950408889634f;
-// 1 / (1 + e^-v) on the hardware's 2^x and reciprocal (each within one unit in the last place)
-__device__ __forceinline__ float sigmoid_d(float v) {
-    return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-v * kLog2E));
-}
 
 struct DeltaRows {
     const int *tok_row, *row_start, *row_len, *row_ctx, *row_slot;
@@ -231,24 +215,6 @@ struct DeltaArgs {
     float *qd, *wk, *kt, *uv, *bm, *s0, *gc;     // scratch, see DeltaScratch
 };
 
-// exp(neg_a * softplus(raw + bias)).  softplus(v) = max(v, 0) + log(1 + e) with e = exp(-|v|), and
-// log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3, by its series to s^15 (the rest is below 2e-9 of the sum): the
-// relative precision stays where e is small - a gate next to one, applied a thousand times over.
-__device__ __forceinline__ float decay_gate(float raw, float bias, float neg_a) {
-    const float v = raw + bias;
-    const float e = __builtin_amdgcn_exp2f(-fabsf(v) * kLog2E);
-    const float s = e * __builtin_amdgcn_rcpf(2.0f + e), s2 = s * s;
-    float c = fmaf(s2, 1.0f / 15.0f, 1.0f / 13.0f);
-    c = fmaf(s2, c, 1.0f / 11.0f);
-    c = fmaf(s2, c, 1.0f / 9.0f);
-    c = fmaf(s2, c, 1.0f / 7.0f);
-    c = fmaf(s2, c, 1.0f / 5.0f);
-    c = fmaf(s2, c, 1.0f / 3.0f);
-    c = fmaf(s2, c, 1.0f);
-    const float sp = fmaf(2.0f * s, c, fmaxf(v, 0.f));
-    return __builtin_amdgcn_exp2f((neg_a * kLog2E) * sp);
-}
-
 // One workgroup per (head, row).  Thread (ng, cl) holds the state rows ng * npt .. + npt of column cl; columns are
 // padded to `pw`, a power of two.  The two sums over state rows (what the key reads, what the query reads) are formed in one
 // pass over the decayed state; the write's share of the read-out is u (k . q).
@@ -351,13 +317,10 @@ __global__ void delta_scan_kernel(DeltaArgs a, int pw) {
 // (r = lane % 16, g = lane / 16).  The contraction index is a label: in step j of a group of 16, slot g stands for
 // index 4 g + j, so a result can be the next product's operand B where it lies and operand A is a 16-byte read.
 constexpr int kDCh = 64;
-#define MV_DMFMA(acc, a_, b_) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a_, b_, acc, 0, 0, 0)
 
 // scratch per (chunk, head): qd, wk (64 x n16) and kt (n16 x 64) in the order in which the lanes of a wave read them as
 // operand A - tile by tile of 16 x 16, lane (r, g) holding row r, columns 4 g .. + 3 -, uv (64 x p16) and s0 (n16 x p16)
 // as slabs of 16 columns, bm [64][64], gc [n16]
-__device__ __forceinline__ int pad16(int v) { return (v + 15) & ~15; }
-
 constexpr int kIntra = 512;      // threads of the intra kernel: two waves a SIMD, one workgroup a compute unit
 
 __global__ __launch_bounds__(kIntra) void delta_chunk_intra_kernel(DeltaArgs a) {

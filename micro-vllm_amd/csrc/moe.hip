@@ -10,6 +10,10 @@
 //                `first_pass` on have no expert behind them: they stand for the input itself (moe_combine)
 //   moe_route_sigmoid  the `top` largest fp32 logits (ties: the lower index), weights = sigmoid of each chosen
 //                logit, not renormalised
+//   moe_route_grouped  scores = sigmoid of the fp32 logits; experts come in `groups` equal runs of neighbours, a run is
+//                worth the sum of its two largest score + correction, and the `top` largest of score + correction are
+//                chosen within the `keep` best runs (ties: the lower index); their weights are the scores themselves
+//                (without the correction), not renormalised
 //   gated_act_scaled  rows sorted by expert: out = act( f(s g) * (s u) ) with s the weight of the row's (token,
 //                choice) pair - an expert that reads weight * h, formed from the products of h itself (the
 //                projections are linear)
@@ -137,6 +141,84 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const void* h_, i
     }
 }
 
+// One workgroup per token; the choice is one wave's: a lane per group of experts, then a lane per expert in turns.
+template <bool F32>
+__global__ __launch_bounds__(256) void moe_route_grouped_kernel(const void* h_, int64_t ldh, const float* wr,
+                                                                const float* correction, int* ids, float* wts, int n,
+                                                                int E, int groups, int keep, int top) {
+    __shared__ float sc[kMaxExperts], ch[kMaxExperts], worth[kMaxExperts];
+    const int t = blockIdx.x, wv = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    for (int e = wv; e < E; e += 4) {
+        const float* w = wr + (int64_t)e * n;
+        float dot = 0.f;
+        if (F32) {
+            const float* h = (const float*)h_ + (int64_t)t * ldh;
+#pragma unroll 8
+            for (int c = lane; c < n; c += 64) dot = fmaf(h[c], w[c], dot);
+        } else {
+            const uint16_t* h = (const uint16_t*)h_ + (int64_t)t * ldh;
+#pragma unroll 8
+            for (int c = lane; c < n; c += 64) dot = fmaf(bf16_bits_to_f32(h[c]), w[c], dot);
+        }
+        dot = wave_sum(dot);
+        if (lane == 0) {
+            const float s = 1.0f / (1.0f + expf(-dot));
+            sc[e] = s;
+            ch[e] = correction ? s + correction[e] : s;
+        }
+    }
+    __syncthreads();
+    const int per = E / groups;
+    for (int g = threadIdx.x; g < groups; g += 256) {
+        float a = -INFINITY, b = -INFINITY;          // the two largest
+        for (int i = 0; i < per; ++i) {
+            const float v = ch[g * per + i];
+            if (v > a) {
+                b = a;
+                a = v;
+            } else if (v > b) {
+                b = v;
+            }
+        }
+        worth[g] = per > 1 ? a + b : a;
+    }
+    __syncthreads();
+    // a group that `keep` others are ahead of is out: its experts can no longer be chosen, whatever their scores
+    for (int g = threadIdx.x; g < groups; g += 256) {
+        int ahead = 0;
+        for (int o = 0; o < groups; ++o) ahead += worth[o] > worth[g] || (worth[o] == worth[g] && o < g);
+        if (ahead >= keep)
+            for (int i = 0; i < per; ++i) ch[g * per + i] = -INFINITY;
+    }
+    __syncthreads();
+    if (wv > 0) return;
+    for (int k = 0; k < top; ++k) {
+        float bv = -INFINITY;
+        int best = E;
+        for (int e = lane; e < E; e += 64)
+            if (ch[e] > bv) {
+                bv = ch[e];
+                best = e;
+            }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+            const float ov = __shfl_xor(bv, o, 64);
+            const int oe = __shfl_xor(best, o, 64);
+            if (ov > bv || (ov == bv && oe < best)) {
+                bv = ov;
+                best = oe;
+            }
+        }
+        best = best < E ? best : E - 1;              // scores that are not numbers choose nothing: stay in bounds
+        if (lane == 0) {
+            ids[(int64_t)t * top + k] = best;
+            wts[(int64_t)t * top + k] = sc[best];
+            ch[best] = -INFINITY;
+        }
+        __builtin_amdgcn_wave_barrier();
+    }
+}
+
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* ids, int* seg, int* order, int* place, int pairs,
                                                         int E) {
     __shared__ int cnt[kMaxExperts + 1];
@@ -259,6 +341,21 @@ int mv_moe_route_sigmoid(const void* h, int64_t ldh, const float* w_router, int3
     hipStream_t s = (hipStream_t)stream;
     if (f32) hipLaunchKernelGGL(moe_route_kernel<true>, dim3(tokens), dim3(256), 0, s, h, ldh, w_router, (const float*)nullptr, ids, weights, (float*)nullptr, n, experts, top, 1);
     else hipLaunchKernelGGL(moe_route_kernel<false>, dim3(tokens), dim3(256), 0, s, h, ldh, w_router, (const float*)nullptr, ids, weights, (float*)nullptr, n, experts, top, 1);
+    return check_launch();
+}
+
+int mv_moe_route_grouped(const void* h, int64_t ldh, const float* w_router, const float* correction, int32_t* ids,
+                         float* weights, int tokens, int n, int experts, int groups, int keep, int top, int f32,
+                         mv_stream_t stream) {
+    using namespace mv;
+    if (tokens < 0 || n <= 0 || experts <= 0 || experts > kMaxExperts || top <= 0 || top > kMaxTop || groups <= 0 ||
+        experts % groups || keep <= 0 || keep > groups || top > keep * (experts / groups))
+        return MV_ERR_INVALID_ARG;
+    if (tokens == 0) return MV_OK;
+    if (!h || !w_router || !ids || !weights || ldh < n) return MV_ERR_INVALID_ARG;
+    hipStream_t s = (hipStream_t)stream;
+    if (f32) hipLaunchKernelGGL(moe_route_grouped_kernel<true>, dim3(tokens), dim3(256), 0, s, h, ldh, w_router, correction, ids, weights, n, experts, groups, keep, top);
+    else hipLaunchKernelGGL(moe_route_grouped_kernel<false>, dim3(tokens), dim3(256), 0, s, h, ldh, w_router, correction, ids, weights, n, experts, groups, keep, top);
     return check_launch();
 }
 

@@ -24,7 +24,11 @@
 //   window_attn                    softmax attention over the last `window` positions (and, where asked for, the
 //                                  sequence's first `keep_first` positions) with a per-head linear distance
 //                                  penalty and / or a per-head sink in the denominator; optionally a sigmoid gate
-//                                  on every output value
+//                                  on every output value.  `chunked`: over the positions of the token's own chunk
+//                                  of `window` positions instead
+//   qkv_headnorm_rotary_store      biases on q, k and v, an RMS norm with one weight for all heads on each head of q
+//                                  and of k, rotation of both; keys and values into their pages; further columns of
+//                                  the same projection cast to the activation type
 //   qkv_norm_rotary_store          biases on q, k and v, RMS norms over ALL heads of q and of k at once, rotation of
 //                                  both, values mixed with another layer's for the same token; keys and values into
 //                                  their pages
@@ -793,6 +797,103 @@ __global__ __launch_bounds__(1024) void qkv_norm_rotary_store_kernel(float* qkv,
     }
 }
 
+// One wave per (token, `hpw` consecutive units): the H heads of q, the G heads of k, the G heads of v, then the cast columns.
+// A head of q or k gets its bias, an RMS norm over itself (weights qn / kn [d], shared by the heads; NULL: no norm) and the
+// rotation of its first `rot` dimensions (adjacent pairs or halves; the angle is formed in fp64 and brought into one turn
+// there, once for the wave's heads); q stays in place, k goes to the key page.  v gets its bias and goes to the value page.
+// A lane's items are the head's rotated pairs, then its other dimensions; NI: items per lane (d - rot / 2 <= 64 NI).
+template <bool F32, int NI>
+__global__ __launch_bounds__(256) void qkv_headnorm_rotary_store_kernel(float* qkv, int64_t ld, const float* qb,
+                                                                        const float* kb, const float* vb,
+                                                                        const float* qn, const float* kn, float eps,
+                                                                        const double* inv_freq, void* kc_, void* vc_,
+                                                                        PagedRows pr, int T, int H, int G, int d, int dv,
+                                                                        int rot, int adjacent, int hpw, const float* low,
+                                                                        int64_t ldl, void* low_out_, int low_n) {
+    typedef typename ActS<F32>::T T_;
+    T_* kc = (T_*)kc_;
+    T_* vc = (T_*)vc_;
+    const int units = H + 2 * G + (low_n > 0 ? 1 : 0), per = (units + hpw - 1) / hpw;
+    const int64_t wave = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
+    if (wave >= (int64_t)T * per) return;
+    const int t = (int)(wave / per), u0 = (int)(wave % per) * hpw, u1 = u0 + hpw < units ? u0 + hpw : units;
+    float* row = qkv + (int64_t)t * ld;
+    const int pos = pr.tok_pos[t];
+    const int pg = pr.block_table[(int64_t)pr.tok_row[t] * pr.bt_stride + pos / pr.page];
+    const int64_t slot = ((int64_t)pg * pr.page + pos % pr.page) * G;
+    const int half = rot / 2, items = d - half;
+    float cs[NI], sn[NI];
+    if (u0 < H + G) {
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int j = lane + 64 * i;
+            cs[i] = 1.f;
+            sn[i] = 0.f;
+            if (j < half) {
+                const double turns = (double)pos * inv_freq[j] * 0.15915494309189533577;      // angle / 2 pi
+                const float a = (float)((turns - rint(turns)) * 6.283185307179586477);
+                sincosf(a, &sn[i], &cs[i]);
+            }
+        }
+    }
+    for (int u = u0; u < u1; ++u) {
+        if (u < H + G) {
+            const bool isq = u < H;
+            float* x = row + (isq ? (int64_t)u * d : (int64_t)H * d + (int64_t)(u - H) * d);
+            const float* b = isq ? (qb ? qb + (int64_t)u * d : nullptr) : (kb ? kb + (int64_t)(u - H) * d : nullptr);
+            const float* w = isq ? qn : kn;
+            float x0[NI], x1[NI], ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                const int j = lane + 64 * i;
+                x0[i] = x1[i] = 0.f;
+                if (j >= items) continue;
+                const int a0 = j < half ? (adjacent ? 2 * j : j) : half + j;
+                x0[i] = b ? x[a0] + b[a0] : x[a0];
+                ss += x0[i] * x0[i];
+                if (j < half) {
+                    const int a1 = adjacent ? 2 * j + 1 : j + half;
+                    x1[i] = b ? x[a1] + b[a1] : x[a1];
+                    ss += x1[i] * x1[i];
+                }
+            }
+            float inv = 1.f;
+            if (w) inv = 1.0f / sqrtf(wave_sum(ss) / (float)d + eps);
+            T_* dst = kc + (slot + (u - H)) * d;
+#pragma unroll
+            for (int i = 0; i < NI; ++i) {
+                const int j = lane + 64 * i;
+                if (j >= items) continue;
+                const int a0 = j < half ? (adjacent ? 2 * j : j) : half + j;
+                const int a1 = adjacent ? 2 * j + 1 : j + half;
+                float y0 = w ? (x0[i] * inv) * w[a0] : x0[i], y1 = 0.f;
+                if (j < half) {
+                    y1 = w ? (x1[i] * inv) * w[a1] : x1[i];
+                    const float r0 = y0 * cs[i] - y1 * sn[i];
+                    y1 = y1 * cs[i] + y0 * sn[i];
+                    y0 = r0;
+                }
+                if (isq) {
+                    x[a0] = y0;
+                    if (j < half) x[a1] = y1;
+                } else if (pg >= 0) {
+                    ActS<F32>::st(dst + a0, y0);
+                    if (j < half) ActS<F32>::st(dst + a1, y1);
+                }
+            }
+        } else if (u < H + 2 * G) {
+            const int g = u - H - G;
+            const float* x = row + (int64_t)(H + G) * d + (int64_t)g * dv;
+            if (pg >= 0)
+                for (int c = lane; c < dv; c += 64) ActS<F32>::st(vc + (slot + g) * dv + c, vb ? x[c] + vb[g * dv + c] : x[c]);
+        } else {
+            T_* lo = (T_*)low_out_ + (int64_t)t * low_n;
+            for (int c = lane; c < low_n; c += 64) ActS<F32>::st(lo + c, low[(int64_t)t * ldl + c]);
+        }
+    }
+}
+
 // value of channel c at token t under a causal convolution of `taps` taps whose first inputs come from the slot
 __device__ __forceinline__ float conv_at(const float* in, int64_t ldi, const float* state, const float* w,
                                          const StepRows& r, int t, int c, int C, int taps) {
@@ -853,6 +954,13 @@ __global__ __launch_bounds__(256) void conv_qkv_store_kernel(const float* in, in
 
 constexpr int kMaxVC = 4;  // value columns per lane: vdim <= 256
 
+// the first position a query at `pos` sees: `size` positions back (a sliding window), or the start of its own chunk of
+// `size` positions, counted from position 0 of the sequence
+__device__ __forceinline__ int first_visible(int pos, int size, int chunked) {
+    const int lo = chunked ? pos - pos % size : pos - size + 1;
+    return lo > 0 ? lo : 0;
+}
+
 // One workgroup per (token, head).  Its NW waves (4, or 16 when a step has too few tokens to fill the
 // chip otherwise: decoding) take the window's 64-key tiles in turn: a lane scores
 // one key (q from LDS, the key row straight from its page), the wave forms max / sum of the tile and
@@ -866,7 +974,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_kernel(const float* q, in
                                                           const float* slopes, int T, int H, int G, int d, int dv,
                                                           float scale, int window, const int* row_len, int max_len,
                                                           int keep_first, const float* sinks, const float* gate,
-                                                          int64_t ldg) {
+                                                          int64_t ldg, int chunked) {
     typedef typename ActS<F32>::T T_;
     extern __shared__ float lds[];
     if (max_len > 0 && row_len[pr.tok_row[blockIdx.x / H]] > max_len) return;   // the tiled kernel's rows
@@ -882,7 +990,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_kernel(const float* q, in
     const int t = blockIdx.x / H, h = blockIdx.x % H, g = h / (H / G);
     const int pos = pr.tok_pos[t];
     const int* bt = pr.block_table + (int64_t)pr.tok_row[t] * pr.bt_stride;
-    const int lo = pos - window + 1 > 0 ? pos - window + 1 : 0;
+    const int lo = first_visible(pos, window, chunked);
     const float slope = slopes ? slopes[h] : 0.f;
     for (int c = threadIdx.x; c < d; c += 64 * NW) qs[c] = q[(int64_t)t * ldq + (int64_t)h * d + c];
     __syncthreads();
@@ -1010,7 +1118,8 @@ __global__ __launch_bounds__(256) void window_attn_group_kernel(const float* q, 
                                                                 PagedRows pr, const float* slopes, const float* sinks,
                                                                 int H, int G, int d, int dv, float scale, int window,
                                                                 int keep_first, const int* row_len, int max_len,
-                                                                int splits, int vec, const float* gate, int64_t ldg) {
+                                                                int splits, int vec, const float* gate, int64_t ldg,
+                                                                int chunked) {
     typedef typename ActS<F32>::T T_;
     constexpr int VEC = F32 ? 4 : 8;
     extern __shared__ float lds[];
@@ -1035,7 +1144,7 @@ __global__ __launch_bounds__(256) void window_attn_group_kernel(const float* q, 
     __syncthreads();
     const int pos = pr.tok_pos[t];
     const int* bt = pr.block_table + (int64_t)pr.tok_row[t] * pr.bt_stride;
-    const int lo = pos - window + 1 > 0 ? pos - window + 1 : 0;
+    const int lo = first_visible(pos, window, chunked);
     const int kept = keep_first < lo ? keep_first : lo;
     const int nk = (kept + 63) / 64, nw = (pos - lo) / 64 + 1;
     float m[RT], l[RT], slope[RT], acc[RT][8];
@@ -1277,7 +1386,7 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
                                                                PagedRows pr, const int* ch_start, const int* ch_len,
                                                                const float* slopes, int H, int G, float scale,
                                                                int window, int keep_first, const float* sinks,
-                                                               const float* gate, int64_t ldg) {
+                                                               const float* gate, int64_t ldg, int chunked) {
     constexpr int D = KS * 32, DV = CT * 16, SK = D + 8, SV = DV + 8;
     __shared__ __attribute__((aligned(16))) uint16_t Ks[64][SK];
     // values as pairs of neighbouring keys: dword [i][c] = V[2i][c] | V[2i+1][c] << 16, which is how the matrix
@@ -1308,8 +1417,9 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) o[ct] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     const float slope = slopes ? slopes[h] : 0.f;
-    const int klo = p0 - window + 1 > 0 ? p0 - window + 1 : 0, khi = p0 + len - 1;
+    const int klo = first_visible(p0, window, chunked), khi = p0 + len - 1;
     const int wq_lo = p0 + 16 * wv, wq_hi = wq_lo + 15;   // this wave's query positions
+    const int wk_lo = first_visible(wq_lo, window, chunked), qlo = first_visible(qpos, window, chunked);
     // key tiles: those of the kept first positions that the window of the chunk's first query has left behind,
     // then the window's
     const int kt_lo = klo / 64, kt_keep = ((keep_first < klo ? keep_first : klo) + 63) / 64;
@@ -1332,7 +1442,7 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
         }
         __syncthreads();
         // nothing of this tile is visible to the wave
-        if (kbase > wq_hi || (kbase + 63 <= wq_lo - window && kbase >= keep_first)) continue;
+        if (kbase > wq_hi || (kbase + 63 < wk_lo && kbase >= keep_first)) continue;
         f32x4_t sc[4];
 #pragma unroll
         for (int nt = 0; nt < 4; ++nt) {
@@ -1349,7 +1459,7 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int kpos = kbase + 16 * nt + 4 * qd + j;
-                const bool ok = qok && kpos <= qpos && (kpos > qpos - window || kpos < keep_first);
+                const bool ok = qok && kpos <= qpos && (kpos >= qlo || kpos < keep_first);
                 const float v = ok ? sc[nt][j] * scale - slope * (float)(qpos - kpos) : -INFINITY;
                 sc[nt][j] = v;
                 mx = fmaxf(mx, v);
@@ -1795,6 +1905,47 @@ int mv_qkv_norm_rotary_store(float* qkv, int64_t ld, const float* q_bias, const 
     return check_launch();
 }
 
+int mv_qkv_headnorm_rotary_store(float* qkv, int64_t ld, const float* q_bias, const float* k_bias, const float* v_bias,
+                                 const float* q_norm, const float* k_norm, float eps, const double* inv_freq,
+                                 void* k_cache, void* v_cache, const int32_t* tok_row, const int32_t* tok_pos,
+                                 const int32_t* block_table, int bt_stride, int page, int tokens, int heads,
+                                 int kv_heads, int d, int dv, int rot, int adjacent, const float* low, int64_t ldl,
+                                 void* low_out, int low_n, int f32, mv_stream_t stream) {
+    using namespace mv;
+    if (tokens < 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || d <= 0 || dv <= 0 || page <= 0 || rot < 0 ||
+        rot > d || rot % 2 || low_n < 0)
+        return MV_ERR_INVALID_ARG;
+    if (d - rot / 2 > 512) return MV_ERR_UNSUPPORTED;
+    if (tokens == 0) return MV_OK;
+    if (!qkv || ld < (int64_t)(heads + kv_heads) * d + (int64_t)kv_heads * dv || !k_cache || !v_cache || !tok_row ||
+        !tok_pos || !block_table || (rot > 0 && !inv_freq) || (low_n > 0 && (!low || !low_out || ldl < low_n)))
+        return MV_ERR_INVALID_ARG;
+    PagedRows pr{tok_row, tok_pos, block_table, bt_stride, page};
+    const int units = heads + 2 * kv_heads + (low_n > 0 ? 1 : 0);
+    // steps of many tokens: a wave takes eight heads of a token and forms the angles' sines and cosines once for them
+    const int hpw = (int64_t)tokens * units >= 8 * 1024 ? 8 : 1;
+    const int64_t blocks = ((int64_t)tokens * ((units + hpw - 1) / hpw) + 3) / 4;
+    if (blocks > 0x7fffffff) return MV_ERR_UNSUPPORTED;
+    const dim3 grid((unsigned)blocks);
+    hipStream_t s = (hipStream_t)stream;
+    const int items = d - rot / 2;
+#define MV_HEADNORM(F32_, NI_)                                                                                       \
+    hipLaunchKernelGGL((qkv_headnorm_rotary_store_kernel<F32_, NI_>), grid, dim3(256), 0, s, qkv, ld, q_bias, k_bias,   \
+                       v_bias, q_norm, k_norm, eps, inv_freq, k_cache, v_cache, pr, tokens, heads, kv_heads, d, dv, rot, \
+                       adjacent, hpw, low, ldl, low_out, low_n)
+#define MV_HEADNORM_N(F32_)                                                                                          \
+    do {                                                                                                           \
+        if (items <= 64) MV_HEADNORM(F32_, 1);                                                                       \
+        else if (items <= 128) MV_HEADNORM(F32_, 2);                                                                 \
+        else MV_HEADNORM(F32_, 8);                                                                                   \
+    } while (0)
+    if (f32) MV_HEADNORM_N(true);
+    else MV_HEADNORM_N(false);
+#undef MV_HEADNORM_N
+#undef MV_HEADNORM
+    return check_launch();
+}
+
 int mv_window_attn_splits(int tokens, int heads, int kv_heads, int window, int keep_first) {
     using namespace mv;
     if (tokens <= 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || window <= 0 || keep_first < 0) return 1;
@@ -1813,7 +1964,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
                    int page, const float* slopes, int tokens, int heads, int kv_heads, int d, int dv, float scale,
                    int window, int f32, const int32_t* row_len, const int32_t* ch_start, const int32_t* ch_len,
                    int chunks, int max_len, int keep_first, const float* sinks, float* part, int splits,
-                   int short_tokens, const float* gate, int64_t ldg, mv_stream_t stream) {
+                   int short_tokens, const float* gate, int64_t ldg, int chunked, mv_stream_t stream) {
     using namespace mv;
     if (gate && ldg < (int64_t)heads * dv) return MV_ERR_INVALID_ARG;
     if (tokens < 0 || heads <= 0 || kv_heads <= 0 || d <= 0 || dv <= 0 || page <= 0 || window <= 0 ||
@@ -1836,7 +1987,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
 #define MV_WA_TILE(KS_, CT_)                                                                                         \
     hipLaunchKernelGGL((window_attn_tile_kernel<KS_, CT_>), tg, dim3(256), 0, s, q, ldq, (const uint16_t*)k_cache,      \
                        (const uint16_t*)v_cache, (uint16_t*)out, ldo, pr, ch_start, ch_len, slopes, heads, kv_heads, scale, \
-                       window, keep_first, sinks, gate, ldg);                                                                         \
+                       window, keep_first, sinks, gate, ldg, chunked);                                                                \
     skip_len = max_len
         if (d == 64 && dv == 64) { MV_WA_TILE(2, 4); }
         else if (d == 96 && dv == 96) { MV_WA_TILE(3, 6); }
@@ -1844,6 +1995,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
         else if (d == 128 && dv == 64) { MV_WA_TILE(4, 4); }
         else if (d == 64 && dv == 128) { MV_WA_TILE(2, 8); }
         else if (d == 32 && dv == 32) { MV_WA_TILE(1, 2); }
+        else if (d == 64 && dv == 32) { MV_WA_TILE(2, 2); }
 #undef MV_WA_TILE
         // every row of the step was long enough for the tiles: nothing is left for the per-token forms
         if (skip_len > 0 && short_tokens == 0) return check_launch();
@@ -1861,7 +2013,7 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
 #define MV_WA_GROUP(F32_, RT_)                                                                                         \
     hipLaunchKernelGGL((window_attn_group_kernel<F32_, RT_>), gg, dim3(256), glds, s, q, ldq, k_cache, v_cache, out, ldo, \
                        part, pr, slopes, sinks, heads, kv_heads, d, dv, scale, window, keep_first, row_len, skip_len,   \
-                       splits, vec, gate, ldg)
+                       splits, vec, gate, ldg, chunked)
             if (f32) {
                 if (rt == 1) MV_WA_GROUP(true, 1); else if (rt == 2) MV_WA_GROUP(true, 2);
                 else if (rt == 4) MV_WA_GROUP(true, 4); else MV_WA_GROUP(true, 8);
@@ -1883,11 +2035,11 @@ int mv_window_attn(const float* q, int64_t ldq, const void* k_cache, const void*
     const size_t lds = (size_t)(d + 64 * nw + 2 * nw + nw * dv) * sizeof(float);
     if (lds > 64 * 1024) return MV_ERR_UNSUPPORTED;
     if (wide) {
-        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
-        else hipLaunchKernelGGL((window_attn_kernel<false, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
+        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg, chunked);
+        else hipLaunchKernelGGL((window_attn_kernel<false, 16>), grid, dim3(1024), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg, chunked);
     } else {
-        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
-        else hipLaunchKernelGGL((window_attn_kernel<false, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg);
+        if (f32) hipLaunchKernelGGL((window_attn_kernel<true, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg, chunked);
+        else hipLaunchKernelGGL((window_attn_kernel<false, 4>), grid, dim3(256), lds, s, q, ldq, k_cache, v_cache, out, ldo, pr, slopes, tokens, heads, kv_heads, d, dv, scale, window, row_len, skip_len, keep_first, sinks, gate, ldg, chunked);
     }
     return check_launch();
 }

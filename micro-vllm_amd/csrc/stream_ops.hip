@@ -34,6 +34,11 @@
 //   cast_concat:         out = act( [a | b] )   (two fp32 streams side by side as one projection's operand)
 //   gelu_tanh:           out = act( gelu(in) ), the tanh form
 //   scale:               v *= s
+//   layernorm_residual:  x += LN(v) with LN(v) = (v - mean) / sqrt(mean((v - mean)^2) + eps) * w, h = act(x) or, with w2,
+//                        act of a second layer norm of the new x.  v is one sublayer's output; or s times the sum of two
+//                        branches, each first divided by its root mean square and weighted; or the weighted sum of a
+//                        token's routed expert rows (+ a shared expert's row)
+//   layernorm_gather:    out = act( LN(x[idx]) )
 // All arithmetic is fp32 with the library's exact division, square root and tanh.
 #include "common.h"
 
@@ -224,6 +229,18 @@ __global__ __launch_bounds__(256) void relu_squared_kernel(const float* in, int6
     if (c >= n) return;
     const float v = fmaxf(in[(int64_t)row * ldi + c], 0.f);
     Act<F32>::st(out + (int64_t)row * ldo + c, v * v);
+}
+
+// the same, four values a thread (n a multiple of 4, rows aligned)
+template <bool F32>
+__global__ __launch_bounds__(256) void relu_squared4_kernel(const float* in, int64_t ldi, void* out_, int64_t ldo, int n4) {
+    const int row = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
+    if (c >= n4) return;
+    float4 v = reinterpret_cast<const float4*>(in + (int64_t)row * ldi)[c];
+    v = make_float4(fmaxf(v.x, 0.f), fmaxf(v.y, 0.f), fmaxf(v.z, 0.f), fmaxf(v.w, 0.f));
+    v = make_float4(v.x * v.x, v.y * v.y, v.z * v.z, v.w * v.w);
+    if (F32) reinterpret_cast<float4*>((float*)out_ + (int64_t)row * ldo)[c] = v;
+    else reinterpret_cast<uint2*>((uint16_t*)out_ + (int64_t)row * ldo)[c] = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
 }
 
 __global__ __launch_bounds__(256) void softcap_kernel(float* v, int64_t count, float cap) {
@@ -528,6 +545,197 @@ __global__ __launch_bounds__(256) void scale_kernel(float* v, int64_t count, flo
     if (i < count) v[i] *= s;
 }
 
+// ---- layer norm on a sublayer's output ----------------------------------------------------------------
+struct LayernormArgs {
+    const float *y1, *r1, *y2, *r2;      // r1 / r2: weights of the two branches' RMS norms (y2 == NULL: y1 as it is)
+    const int* place;                    // experts: rows of y1 the token's choices lie in, [rows, top]
+    const float* wts;                    // [rows, top]
+    const float *w, *w2;
+    int64_t ld1, ld2, ldx, ldh;
+    float s, eps;
+    float* x;
+    void* h;
+    int n, top;
+};
+
+// The row in registers, VEC (4: every row 16-byte aligned, n a multiple of 4; or 1) values a thread and turn, NV turns.
+template <bool F32, int VEC, int NV>
+__global__ __launch_bounds__(1024) void layernorm_residual_kernel(LayernormArgs a) {
+    typedef typename Act<F32>::T T;
+    __shared__ float red[16], red2[16];
+    const int row = blockIdx.x, tid = threadIdx.x, NT = blockDim.x, cnt = a.n / VEC;
+    auto load = [&](const float* p, int c, float (&o)[VEC]) {
+        if (VEC == 4) {
+            const float4 q = reinterpret_cast<const float4*>(p)[c];
+            o[0] = q.x; o[VEC > 1 ? 1 : 0] = q.y; o[VEC > 2 ? 2 : 0] = q.z; o[VEC > 3 ? 3 : 0] = q.w;
+        } else {
+            o[0] = p[c];
+        }
+    };
+    float v[NV][VEC], xv[NV][VEC];
+    float* xr = a.x + (int64_t)row * a.ldx;
+    const float* y1 = a.y1 + (int64_t)row * a.ld1;
+    const float* y2 = a.y2 ? a.y2 + (int64_t)row * a.ld2 : nullptr;
+    const bool branches = y2 && !a.place;
+    float u[NV][VEC];                    // the second branch
+    float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = tid + NT * i;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[i][j] = u[i][j] = xv[i][j] = 0.f;
+        if (c >= cnt) continue;
+        load(xr, c, xv[i]);
+        if (a.place) {
+            if (y2) load(y2, c, v[i]);
+        } else {
+            load(y1, c, v[i]);
+            if (y2) load(y2, c, u[i]);
+        }
+    }
+    if (a.place) {
+        constexpr int kB = 4;            // expert rows in flight together
+        for (int k0 = 0; k0 < a.top; k0 += kB) {
+            const float* e[kB];
+            float ew[kB];
+#pragma unroll
+            for (int k = 0; k < kB; ++k) {
+                const int64_t at = (int64_t)row * a.top + (k0 + k < a.top ? k0 + k : k0);
+                e[k] = a.y1 + (int64_t)a.place[at] * a.ld1;
+                ew[k] = k0 + k < a.top ? a.wts[at] : 0.f;
+            }
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                const int c = tid + NT * i;
+                if (c >= cnt) continue;
+                float q[kB][VEC];
+#pragma unroll
+                for (int k = 0; k < kB; ++k) load(e[k], c, q[k]);
+#pragma unroll
+                for (int k = 0; k < kB; ++k)
+#pragma unroll
+                    for (int j = 0; j < VEC; ++j) v[i][j] = fmaf(ew[k], q[k][j], v[i][j]);
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            s1 += branches ? v[i][j] * v[i][j] : v[i][j];
+            s2 += u[i][j] * u[i][j];
+        }
+    if (branches) {
+        s1 = wave_sum(s1);
+        s2 = wave_sum(s2);
+        if ((tid & 63) == 0) {
+            red[tid >> 6] = s1;
+            red2[tid >> 6] = s2;
+        }
+        __syncthreads();
+        s1 = s2 = 0.f;
+        for (int i = 0; i < NT / 64; ++i) {
+            s1 += red[i];
+            s2 += red2[i];
+        }
+        __syncthreads();
+        const float i1 = 1.0f / sqrtf(s1 / (float)a.n + a.eps), i2 = 1.0f / sqrtf(s2 / (float)a.n + a.eps);
+        s1 = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int c = tid + NT * i;
+            if (c >= cnt) continue;
+            float w1[VEC], w2[VEC];
+            load(a.r1, c, w1);
+            load(a.r2, c, w2);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) {
+                v[i][j] = a.s * ((v[i][j] * i1) * w1[j] + (u[i][j] * i2) * w2[j]);
+                s1 += v[i][j];
+            }
+        }
+    }
+    // mean, then the squared deviations from it; the row stays in registers
+    const float mean = block_sum(s1, red) / (float)a.n;
+    float sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            v[i][j] = tid + NT * i < cnt ? v[i][j] - mean : 0.f;
+            sq += v[i][j] * v[i][j];
+        }
+    const float inv = 1.0f / sqrtf(block_sum(sq, red) / (float)a.n + a.eps);
+    float sx = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = tid + NT * i;
+        if (c >= cnt) continue;
+        float w[VEC];
+        load(a.w, c, w);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            xv[i][j] += (v[i][j] * inv) * w[j];
+            sx += xv[i][j];
+        }
+        if (VEC == 4) reinterpret_cast<float4*>(xr)[c] = make_float4(xv[i][0], xv[i][VEC > 1 ? 1 : 0], xv[i][VEC > 2 ? 2 : 0], xv[i][VEC > 3 ? 3 : 0]);
+        else xr[c] = xv[i][0];
+    }
+    float inv2 = 1.f, mean2 = 0.f;
+    if (a.w2) {
+        mean2 = block_sum(sx, red) / (float)a.n;
+        sq = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) {
+                const float d = tid + NT * i < cnt ? xv[i][j] - mean2 : 0.f;
+                sq += d * d;
+            }
+        inv2 = 1.0f / sqrtf(block_sum(sq, red) / (float)a.n + a.eps);
+    }
+    if (!a.h) return;
+    T* h = (T*)a.h + (int64_t)row * a.ldh;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = tid + NT * i;
+        if (c >= cnt) continue;
+        float o[VEC];
+        if (a.w2) {
+            load(a.w2, c, o);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) o[j] = ((xv[i][j] - mean2) * inv2) * o[j];
+        } else {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) o[j] = xv[i][j];
+        }
+        if (VEC == 4) {
+            const float o1 = o[VEC > 1 ? 1 : 0], o2 = o[VEC > 2 ? 2 : 0], o3 = o[VEC > 3 ? 3 : 0];
+            if (F32) reinterpret_cast<float4*>(h)[c] = make_float4(o[0], o1, o2, o3);
+            else reinterpret_cast<uint2*>(h)[c] = make_uint2(pack_bf16x2(o[0], o1), pack_bf16x2(o2, o3));
+        } else {
+            Act<F32>::st(h + c, o[0]);
+        }
+    }
+}
+
+template <bool F32>
+__global__ __launch_bounds__(256) void layernorm_gather_kernel(const float* x, int64_t ldx, const int* idx, const float* w,
+                                                               float eps, void* out_, int64_t ldo, int n) {
+    typedef typename Act<F32>::T T;
+    __shared__ float red[4];
+    T* out = (T*)out_;
+    const int row = blockIdx.x;
+    const float* a = x + (int64_t)(idx ? idx[row] : row) * ldx;
+    float s = 0.f;
+    for (int c = threadIdx.x; c < n; c += 256) s += a[c];
+    const float mean = block_sum(s, red) / (float)n;
+    s = 0.f;
+    for (int c = threadIdx.x; c < n; c += 256) s += (a[c] - mean) * (a[c] - mean);
+    const float inv = 1.0f / sqrtf(block_sum(s, red) / (float)n + eps);
+    for (int c = threadIdx.x; c < n; c += 256) Act<F32>::st(out + (int64_t)row * ldo + c, ((a[c] - mean) * inv) * w[c]);
+}
+
 }  // namespace mv
 
 extern "C" {
@@ -649,6 +857,12 @@ int mv_relu_squared(const float* in, int64_t ldi, void* out, int64_t ldo, int ro
     if (rows == 0) return MV_OK;
     if (!in || !out || ldi < n || ldo < n) return MV_ERR_INVALID_ARG;
     hipStream_t s = (hipStream_t)stream;
+    if (n % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && aligned16(in) && aligned16(out)) {
+        const dim3 g4(rows, (n / 4 + 255) / 256);
+        if (f32) hipLaunchKernelGGL(relu_squared4_kernel<true>, g4, dim3(256), 0, s, in, ldi, out, ldo, n / 4);
+        else hipLaunchKernelGGL(relu_squared4_kernel<false>, g4, dim3(256), 0, s, in, ldi, out, ldo, n / 4);
+        return check_launch();
+    }
     const dim3 grid(rows, (n + 255) / 256);
     if (f32) hipLaunchKernelGGL(relu_squared_kernel<true>, grid, dim3(256), 0, s, in, ldi, out, ldo, n);
     else hipLaunchKernelGGL(relu_squared_kernel<false>, grid, dim3(256), 0, s, in, ldi, out, ldo, n);
@@ -814,6 +1028,56 @@ int mv_scale(float* v, int64_t count, float factor, mv_stream_t stream) {
     if (!v) return MV_ERR_INVALID_ARG;
     hipLaunchKernelGGL(scale_kernel, dim3((unsigned)((count + 255) / 256)), dim3(256), 0, (hipStream_t)stream, v, count,
                        factor);
+    return check_launch();
+}
+
+int mv_layernorm_residual(const float* y1, int64_t ld1, const float* r1, const float* y2, int64_t ld2, const float* r2,
+                          float s, const int32_t* place, const float* weights, int top, const float* w, float eps,
+                          const float* next_w, float* x, int64_t ldx, void* h, int64_t ldh, int rows, int n, int f32,
+                          mv_stream_t stream) {
+    using namespace mv;
+    if (rows < 0 || n <= 0) return MV_ERR_INVALID_ARG;
+    if (rows == 0) return MV_OK;
+    if (!y1 || !w || !x || ld1 < n || (y2 && ld2 < n) || ldx < n || (h && ldh < n) || (next_w && !h)) return MV_ERR_INVALID_ARG;
+    if (place ? (!weights || top <= 0 || r1 || r2) : (y2 ? (!r1 || !r2) : (r1 || r2))) return MV_ERR_INVALID_ARG;
+    LayernormArgs a;
+    a.y1 = y1; a.r1 = r1; a.y2 = y2; a.r2 = r2; a.place = place; a.wts = weights; a.w = w; a.w2 = next_w;
+    a.ld1 = ld1; a.ld2 = ld2; a.ldx = ldx; a.ldh = ldh; a.s = s; a.eps = eps; a.x = x; a.h = h; a.n = n; a.top = top;
+    auto al = [](const void* p) { return !p || aligned16(p); };
+    const bool even = n % 4 == 0 && ld1 % 4 == 0 && ldx % 4 == 0 && (!h || ldh % 4 == 0) && (!y2 || ld2 % 4 == 0) && al(y1) &&
+                      al(y2) && al(r1) && al(r2) && al(w) && al(next_w) && al(x) && al(h);
+    const int vec = even ? 4 : 1;
+    // a row of a short step has its workgroup to itself on a compute unit: more threads, fewer values each
+    int nt = rows > 512 ? 256 : 1024;
+    while (nt > 64 && n <= vec * (nt / 2)) nt /= 2;
+    while (nt < 1024 && n > vec * nt * 4) nt *= 2;
+    const int turns = (n + vec * nt - 1) / (vec * nt);
+    hipStream_t st = (hipStream_t)stream;
+#define MV_LAYERNORM(VEC_, NV_)                                                                                      \
+    do {                                                                                                             \
+        if (f32) hipLaunchKernelGGL((layernorm_residual_kernel<true, VEC_, NV_>), dim3(rows), dim3(nt), 0, st, a);    \
+        else hipLaunchKernelGGL((layernorm_residual_kernel<false, VEC_, NV_>), dim3(rows), dim3(nt), 0, st, a);       \
+    } while (0)
+    if (even && turns == 1) MV_LAYERNORM(4, 1);
+    else if (even && turns == 2) MV_LAYERNORM(4, 2);
+    else if (even && turns <= 4) MV_LAYERNORM(4, 4);
+    else if (!even && turns == 1) MV_LAYERNORM(1, 1);
+    else if (!even && turns <= 4) MV_LAYERNORM(1, 4);
+    else if (!even && turns <= 16) MV_LAYERNORM(1, 16);
+    else return MV_ERR_UNSUPPORTED;
+#undef MV_LAYERNORM
+    return check_launch();
+}
+
+int mv_layernorm_gather(const float* x, int64_t ldx, const int32_t* idx, const float* w, float eps, void* out,
+                        int64_t ldo, int rows, int n, int f32, mv_stream_t stream) {
+    using namespace mv;
+    if (rows < 0 || n <= 0) return MV_ERR_INVALID_ARG;
+    if (rows == 0) return MV_OK;
+    if (!x || !w || !out || ldx < n || ldo < n) return MV_ERR_INVALID_ARG;
+    hipStream_t s = (hipStream_t)stream;
+    if (f32) hipLaunchKernelGGL(layernorm_gather_kernel<true>, dim3(rows), dim3(256), 0, s, x, ldx, idx, w, eps, out, ldo, n);
+    else hipLaunchKernelGGL(layernorm_gather_kernel<false>, dim3(rows), dim3(256), 0, s, x, ldx, idx, w, eps, out, ldo, n);
     return check_launch();
 }
 

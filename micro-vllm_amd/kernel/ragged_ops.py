@@ -265,13 +265,15 @@ def qk_rotary_store(qk, q_bias, k_bias, k_cache, v_cache, inv_freq, step, heads:
 
 def window_attn(q, k_cache, v_cache, out, step, slopes, heads: int, kv_heads: int, d: int, dv: int,
                 scale: float, window: int, tiled: bool = True, keep_first: int = 0, sinks=None, part=None, splits: int = 0,
-                gate=None):
+                gate=None, chunked: bool = False):
     """`tiled`: rows of more than SCAN_SEQ_MAX tokens go to the matrix-core kernel where it applies (bf16,
     the head shapes it is built for); False keeps every token on the plain kernel.  `keep_first`: positions below it
     stay visible behind the window; `sinks` [heads]: exp(sink) joins each head's denominator.  `part` (fp32, at least
     tokens * heads * splits * (dv + 2) values, `splits` from window_attn_splits): the tokens the matrix-core kernel
     does not take run the kernel that reads every key once for all query heads of its key/value head and cuts the keys
-    into `splits` pieces.  `gate` [tokens, heads * dv] fp32: the output is multiplied by its sigmoid."""
+    into `splits` pieces.  `gate` [tokens, heads * dv] fp32: the output is multiplied by its sigmoid.  `chunked`: a token
+    sees its own chunk of `window` positions up to itself, chunks counted from position 0 of its sequence, instead of the
+    last `window` positions."""
     assert gate is None or gate.shape == (q.shape[0], heads * dv)
     assert part is None or (splits >= 1 and part.is_contiguous() and part.numel() >= q.shape[0] * heads * splits * (dv + 2))
     assert sinks is None or (sinks.numel() == heads and sinks.is_contiguous())
@@ -290,7 +292,7 @@ def window_attn(q, k_cache, v_cache, out, step, slopes, heads: int, kv_heads: in
         step.n_chunks if tiled else 0, SCAN_SEQ_MAX, int(keep_first), None if sinks is None else _f32(sinks).data_ptr(),
         None if part is None else _f32(part).data_ptr(), int(splits) if part is not None else 0,
         int(getattr(step, "short_tokens", -1)) if tiled else -1, None if gate is None else _f32(gate).data_ptr(),
-        0 if gate is None else _ld(gate), nv.stream_ptr()))
+        0 if gate is None else _ld(gate), int(chunked), nv.stream_ptr()))
 
 
 def window_attn_splits(tokens: int, heads: int, kv_heads: int, window: int, keep_first: int = 0) -> int:
@@ -818,3 +820,110 @@ def delta_rule(qkv, gate_in, z, beta, dt_bias, a_log, norm, state, out, step, kv
         step.ch_len.data_ptr() if chunks else None, step.row_ch0.data_ptr() if chunks else None,
         step.row_nch.data_ptr() if chunks else None, chunks, SCAN_SEQ_MAX,
         int(getattr(step, "short_tokens", -1)) if chunks else -1, _is_f32(out), nv.stream_ptr()))
+
+
+# ---------------------------------------------------------------------------------------------------------
+# Per-head norms with rotation, gated linear attention, group-limited routing, layer norm on sublayer outputs
+# (csrc/seq_mix.hip, gla.hip, moe.hip, stream_ops.hip)
+
+def qkv_headnorm_rotary_store(qkv, k_cache, v_cache, step, heads: int, kv_heads: int, d: int, dv: int, inv_freq, rot: int,
+                              eps: float, q_bias=None, k_bias=None, v_bias=None, q_norm=None, k_norm=None,
+                              adjacent: bool = False, low=None, low_out=None):
+    """qkv [T, heads*d + kv_heads*(d + dv)] fp32 = q | k | v of one projection.  Every head of q and k gets its bias, an RMS
+    norm over itself (weights q_norm / k_norm [d]; None: no norm) and the rotation of its first `rot` dimensions; q stays
+    in place, k goes to its page.  v gets its bias and goes to its page.  low_out [T, n] = act(low [T, n])."""
+    tokens = qkv.shape[0]
+    page = k_cache.shape[1]
+    assert qkv.shape[1] == (heads + kv_heads) * d + kv_heads * dv and step.tokens == tokens
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dtype == v_cache.dtype
+    assert k_cache.shape[1:] == (page, kv_heads, d) and v_cache.shape == (k_cache.shape[0], page, kv_heads, dv)
+    assert int(step.max_page) < k_cache.shape[0] and page == step.page
+    for t, n in ((q_bias, heads * d), (k_bias, kv_heads * d), (v_bias, kv_heads * dv), (q_norm, d), (k_norm, d)):
+        assert t is None or (t.numel() == n and t.is_contiguous())
+    assert rot == 0 or (inv_freq.is_cuda and inv_freq.dtype == torch.float64 and inv_freq.numel() == rot // 2)
+    assert low is None or (low.shape == low_out.shape and low.shape[0] == tokens and low_out.is_contiguous()
+                           and low_out.dtype == k_cache.dtype)
+    p = lambda t: None if t is None else _f32(t).data_ptr()   # noqa: E731
+    nv.check("mv_qkv_headnorm_rotary_store", nv.lib().mv_qkv_headnorm_rotary_store(
+        _f32(qkv).data_ptr(), _ld(qkv), p(q_bias), p(k_bias), p(v_bias), p(q_norm), p(k_norm), float(eps),
+        None if rot == 0 else inv_freq.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), step.tok_row.data_ptr(),
+        step.tok_pos.data_ptr(), step.block_table.data_ptr(), step.block_table.stride(0), page, tokens, heads, kv_heads, d,
+        dv, rot, int(adjacent), p(low), 0 if low is None else _ld(low), None if low is None else low_out.data_ptr(),
+        0 if low is None else low.shape[1], _is_f32(k_cache), nv.stream_ptr()))
+
+
+def gated_linear_attn(q, k, v, z, z_bias, gate, norm, state, out, step, heads: int, n: int, p: int, tau: float, eps: float,
+                      q_scale: float = 1.0, chunked: bool = True):
+    """S_t = diag(sigmoid(z_t + z_bias)^(1 / tau)) S_(t-1) + k_t v_t^T, o_t = S_t^T (q_t q_scale); out [T, heads*p] =
+    act(unit-RMS per head of o * norm * silu(gate)); state [slots, heads, n, p] fp32.  Rows of up to SCAN_SEQ_MAX tokens run
+    token by token; longer rows in chunks of 64 unless `chunked` is False or the head's shape is beyond that form."""
+    tokens = q.shape[0]
+    assert q.shape == k.shape == z.shape == (tokens, heads * n) and step.tokens == tokens
+    assert v.shape == gate.shape == out.shape == (tokens, heads * p)
+    assert z_bias is None or (z_bias.numel() == heads * n and z_bias.is_contiguous())
+    assert norm.numel() == p and norm.is_contiguous()
+    assert state.is_contiguous() and state.shape[1:] == (heads, n, p) and int(step.max_slot) < state.shape[0]
+    L = nv.lib()
+    chunks = step.n_chunks if chunked and L.mv_gated_linear_chunked_ok(n, p) else 0
+    scratch = None
+    if chunks:
+        scratch = torch.empty(chunks * heads * L.mv_gated_linear_scratch_floats(n, p), dtype=torch.float32, device=q.device)
+    nv.check("mv_gated_linear_attn", L.mv_gated_linear_attn(
+        _f32(q).data_ptr(), _ld(q), _f32(k).data_ptr(), _ld(k), _f32(v).data_ptr(), _ld(v), _f32(z).data_ptr(), _ld(z),
+        None if z_bias is None else _f32(z_bias).data_ptr(), _f32(gate).data_ptr(), _ld(gate), _f32(norm).data_ptr(),
+        _f32(state).data_ptr(), out.data_ptr(), _ld(out), step.row_start.data_ptr(), step.row_len.data_ptr(),
+        step.row_ctx.data_ptr(), step.row_slot.data_ptr(), step.rows, heads, n, p, float(q_scale), 1.0 / float(tau),
+        float(eps), None if scratch is None else scratch.data_ptr(), step.ch_start.data_ptr() if chunks else None,
+        step.ch_len.data_ptr() if chunks else None, step.row_ch0.data_ptr() if chunks else None,
+        step.row_nch.data_ptr() if chunks else None, chunks, SCAN_SEQ_MAX,
+        int(getattr(step, "short_tokens", -1)) if chunks else -1, _is_f32(out), nv.stream_ptr()))
+
+
+def moe_route_grouped(h, w_router, correction, ids, weights, groups: int, keep: int):
+    """Scores = sigmoid of the router outputs; the `top` largest of score + correction within the `keep` best of `groups`
+    equal runs of experts (a run is worth the sum of its two largest) are chosen; the weights are their scores."""
+    tokens, n = h.shape
+    E, top = w_router.shape[0], ids.shape[1]
+    assert h.stride(1) == 1 and w_router.shape == (E, n) and w_router.is_contiguous()
+    assert ids.shape == (tokens, top) and weights.shape == (tokens, top) and ids.is_contiguous()
+    assert weights.is_contiguous() and ids.dtype == torch.int32
+    assert correction is None or (correction.numel() == E and correction.is_contiguous())
+    nv.check("mv_moe_route_grouped", nv.lib().mv_moe_route_grouped(
+        h.data_ptr(), _ld(h), _f32(w_router).data_ptr(), None if correction is None else _f32(correction).data_ptr(),
+        ids.data_ptr(), _f32(weights).data_ptr(), tokens, n, E, int(groups), int(keep), top, _is_f32(h), nv.stream_ptr()))
+
+
+def layernorm_residual(x, y1, w, eps: float, h=None, branch=None, place=None, weights=None, shared=None, next_w=None):
+    """x += LN(v; w); h (optional) = act(x), or with `next_w` act(LN(x; next_w)).  v = y1; with `branch` = (r1, y2, r2, s):
+    s * (unit_rms(y1) * r1 + unit_rms(y2) * r2); with `place` [rows * top] and `weights` [rows, top]: the weighted sum of
+    each row's rows of y1 (+ its row of `shared`)."""
+    rows, n = x.shape
+    r1 = y2 = r2 = None
+    s, top = 1.0, 0
+    assert w.numel() == n and w.is_contiguous() and (h is None or h.shape == (rows, n))
+    assert next_w is None or (h is not None and next_w.numel() == n and next_w.is_contiguous())
+    if place is not None:
+        top, y2 = weights.shape[1], shared
+        assert branch is None and weights.shape == (rows, top) and weights.is_contiguous() and place.numel() == rows * top
+        assert y1.shape == (rows * top, n)
+    else:
+        assert y1.shape == (rows, n) and shared is None
+        if branch is not None:
+            r1, y2, r2, s = branch
+            assert all(r.numel() == n and r.is_contiguous() for r in (r1, r2))
+    assert y2 is None or y2.shape == (rows, n)
+    p = lambda t: None if t is None else _f32(t).data_ptr()   # noqa: E731
+    nv.check("mv_layernorm_residual", nv.lib().mv_layernorm_residual(
+        _f32(y1).data_ptr(), _ld(y1), p(r1), p(y2), 0 if y2 is None else _ld(y2), p(r2), float(s),
+        None if place is None else _i32(place).data_ptr(), p(weights), top, _f32(w).data_ptr(), float(eps), p(next_w),
+        _f32(x).data_ptr(), _ld(x), None if h is None else h.data_ptr(), 0 if h is None else _ld(h), rows, n,
+        0 if h is None else _is_f32(h), nv.stream_ptr()))
+
+
+def layernorm_gather(x, idx, w, eps: float, out):
+    rows, n = out.shape
+    assert x.shape[1] == n and w.numel() == n and w.is_contiguous()
+    assert (x.shape[0] == rows) if idx is None else idx.numel() == rows
+    nv.check("mv_layernorm_gather", nv.lib().mv_layernorm_gather(
+        _f32(x).data_ptr(), _ld(x), None if idx is None else _i32(idx).data_ptr(), _f32(w).data_ptr(), float(eps),
+        out.data_ptr(), _ld(out), rows, n, _is_f32(out), nv.stream_ptr()))

@@ -7,7 +7,7 @@ A family = (configuration reader, model object, runner and cache manager the eng
   "ragged" - stacks with an fp32 residual stream whose layers are listed one by one (recurrent
              mixers, windowed or latent attention, dense or routed feed-forwards), run step by step
              over ragged batches (RaggedRunner / HybridCacheManager): Pagazen, Fagunex, Nesisun, Solopel,
-             Dugazen.
+             Dugazen, Sizizen.
 """
 from typing import Callable, Dict
 
@@ -64,11 +64,21 @@ def _load_dugazen(config_json, files, name):
     return DugazenModel(cfg, files)
 
 
+def _load_sizizen(config_json, files, name):
+    from .sizizen import SizizenConfig, SizizenModel, tensor_shapes
+    cfg = SizizenConfig.from_json(config_json, name)
+    for tensor, shape in tensor_shapes(cfg).items():
+        if tensor not in files:
+            raise KeyError(f"tensor {tensor!r} {shape} is not in the checkpoint")
+    return SizizenModel(cfg, files)
+
+
 register("Pagazen", _load_pagazen)
 register("Fagunex", _load_fagunex)
 register("Nesisun", _load_nesisun)
 register("Solopel", _load_solopel)
 register("Dugazen", _load_dugazen)
+register("Sizizen", _load_sizizen)
 
 
 def loader_for(config_json: dict):
