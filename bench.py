@@ -104,6 +104,15 @@ def parse():
                          "line of its own")
     ap.add_argument("--dugazen-widths", default="1024,2048,4096")
     ap.add_argument("--dugazen-kernels", action="store_true", help="with --dugazen: per-op times of one step on stderr")
+    ap.add_argument("--sizizen", action="store_true",
+                    help="instead of the default workload: prefill and decode throughput of the Sizizen design (attention "
+                         "within chunks beside gated linear attention in every layer, layer norms on sublayer outputs, "
+                         "dense or group-routed feed-forwards; random weights) at a few widths beside the family's closest "
+                         "designs at equal width, depth and feed-forward parameters: Pagazen with a parallel mixer in "
+                         "every layer (windowed attention beside retention) and Fagunex (a gate per state row, routed "
+                         "experts); one JSON line of its own")
+    ap.add_argument("--sizizen-widths", default="1024,2048,4096")
+    ap.add_argument("--sizizen-kernels", action="store_true", help="with --sizizen: per-op times of one step on stderr")
     return ap.parse_args()
 
 
@@ -804,6 +813,44 @@ def dugazen_compare(args, dev):
                       "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "n_gpus": 1, "rows": rows}), flush=True)
 
 
+def sizizen_compare(args, dev):
+    """Prefill (one prompt of --ctx tokens) and decode (bs 1 and 8 at context --ctx) of the Sizizen design - once with
+    dense feed-forwards (gate, up, down of 4 x width), once with every one routed (16 experts in four groups of which two
+    are kept, four experts used, beside a shared one: up and down of 6 x width active) - beside Pagazen and Fagunex, all
+    through InferenceEngine.run_ragged.  Random weights, 4 layers, vocabulary 32000, 128-wide heads, a low-rank map of 128.
+    Pagazen: a parallel mixer in every layer with the same heads, a window as long as Sizizen's chunks (1024), the same
+    128 x 128 states, up and down with 6 x width; Fagunex: three gated recurrences and one latent attention, routed
+    experts with gate, up and down of 4 x width active."""
+    import micro_vllm_amd  # noqa: F401
+    from micro_vllm_amd.core.engine import InferenceEngine
+    from micro_vllm_amd.models import fagunex, pagazen, sizizen
+
+    def pagazen_parallel(width):
+        cfg = pagazen.bench_config(width, layers, ff_mult=6, every=1)
+        for layer in cfg.layers:
+            layer["mixer"]["right"]["vdim"] = 128
+        return pagazen.build_random_model(cfg, 1)
+
+    S, layers, rows = args.ctx, 4, []
+    for width in [int(w) for w in args.sizizen_widths.split(",")]:
+        row = {"width": width, "layers": layers, "ctx": S}
+        for name, make in (("sizizen_dense", lambda: sizizen.build_random_model(sizizen.bench_config(width, layers), 1, rank=128)),
+                           ("pagazen", lambda: pagazen_parallel(width)),
+                           ("sizizen_routed", lambda: sizizen.build_random_model(
+                               sizizen.bench_config(width, layers, ff_mult=6, moe_every=1), 1, rank=128)),
+                           ("fagunex", lambda: fagunex.build_random_model(fagunex.bench_config(width, layers), 1))):
+            model = make()
+            eng = InferenceEngine(model=model, max_batch_size=8, max_prefill_tokens=S, n_blocks=9 * (S // 64 + 4),
+                                  max_tokens=S + 256, state_slots=9)
+            row.update(_ragged_engine_row(eng, model.config, S, name, args.sizizen_kernels, width))
+            del eng, model
+            torch.cuda.empty_cache()
+        log(f"[bench] {row}")
+        rows.append(row)
+    print(json.dumps({"metric": "Sizizen beside Pagazen and Fagunex (ragged family): prefill and decode tokens/s at equal size",
+                      "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "n_gpus": 1, "rows": rows}), flush=True)
+
+
 def pagazen_kernel_table(eng, ids, width):
     """Per-op time of one prefill step and one single-token step (rocprof-free: HIP events around each
     wrapper call), printed on stderr."""
@@ -817,7 +864,8 @@ def pagazen_kernel_table(eng, ids, width):
              "latent_attn", "moe_route", "moe_plan", "moe_combine", "embed_pair", "add_rmsnorm", "rmsnorm_gather",
              "gated_act", "qk_rotary_store", "moe_route_scored", "gated_residual_norm", "cast_concat", "gelu_tanh",
              "scale_", "conv_taps", "conv_qkv_store", "diff_attn", "moe_route_sigmoid", "gated_act_scaled", "qkv_norm_rotary_store",
-             "delta_prep", "delta_rule"]
+             "delta_prep", "delta_rule", "qkv_headnorm_rotary_store", "gated_linear_attn", "moe_route_grouped",
+             "layernorm_residual", "layernorm_gather"]
     saved = {n: getattr(ops, n) for n in names}
     saved_call = ops.AnyLinear.__call__
 
@@ -958,6 +1006,9 @@ def main():
     if args.dugazen:
         assert world == 1, "--dugazen runs on one GPU"
         return dugazen_compare(args, dev)
+    if args.sizizen:
+        assert world == 1, "--sizizen runs on one GPU"
+        return sizizen_compare(args, dev)
     peers = world > 1                 # ranks to synchronise with
     if args.as_rank_of:
         assert world == 1, "--as-rank-of runs one process"
