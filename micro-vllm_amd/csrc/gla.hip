@@ -9,8 +9,8 @@
 //                     G_t = alpha_1 * ... * alpha_t per state row (t counted within the chunk):
 //                       O = (G * Q) S0 + B V,  B[t][s] = sum_i q_t[i] k_s[i] (G_t / G_s)[i]  (s <= t)
 //                       S_end = diag(G_end) S0 + ((G_end / G) * K)^T V
-//     keys    per (chunk, head, state row): (G_end / G) * K in the order the carry's lanes read it, and G_end
-//     carry   per (row, head, 16 x 16 tile of the state), one wave each: the state from chunk to chunk
+//     state   per (chunk, head): G_end and what the chunk adds to the state, ((G_end / G) * K)^T V
+//     carry   per (row, head, value of the state): the state each chunk starts from, and the one the row leaves
 //     out     per (chunk, head): B, O, its norm and gate
 // The quotients are never formed: a chunk is four blocks of 16 tokens, G_t / G_s is the product of the gates from the
 // start of t's block to t, of whole blocks in between, and from s to the end of s's block - products of numbers in
@@ -30,11 +30,11 @@ struct GlaArgs {
     float* state;           // [slots, H, n, p]
     void* out;              // [T, ldo] activation type
     const int *row_start, *row_len, *row_ctx, *row_slot;
-    int H, n, p, max_len, vec_in, vec_out;
+    int H, n, p, max_len, vec_in, vec_v, vec_out;
     float eps, q_scale, neg_inv_tau;
     // chunks of long rows
     const int *ch_start, *ch_len, *row_ch0, *row_nch;
-    float *kt, *s0, *gc;    // per (chunk, head): 64 x N, N x P, N with N, P the padded sizes
+    float *s0, *gc;         // per (chunk, head): N x P (16 x 16 tiles, a tile's lane (r, g) rows 4 g .. + 3 of column r), N
 };
 
 // sigmoid(z + bias)^(1 / tau) = exp(-softplus(-(z + bias)) / tau)
@@ -112,112 +112,126 @@ __global__ void gla_scan_kernel(GlaArgs a, int pw) {
         if (i < mine) sp[(int64_t)i * p] = S[i];
 }
 
-// Thread per (chunk, head, state row): the keys of the chunk's tokens times the gates behind them, walking backwards.
-// kt holds 16 x 16 tiles (state rows x tokens), tile by tile; in a tile lane (r, g) reads state row r, tokens 4 g .. + 3.
-__global__ __launch_bounds__(256) void gla_chunk_keys_kernel(GlaArgs a) {
-    const int N = pad16(a.n), ch = blockIdx.y, e = blockIdx.x * 256 + threadIdx.x;
-    if (e >= a.H * N) return;
-    const int h = e / N, i = e - h * N;
+// One workgroup per (head, chunk).  A wave takes 16 state rows at a time: lane (r, g) holds row r's keys and gates of the
+// tokens 4 g .. + 3 of each block of 16, the products of the gates behind a token come from its own four, from the lanes
+// with larger g and from the blocks behind, and the weighted keys are the matrix product's operand where they lie; the
+// values lie in LDS.
+__global__ __launch_bounds__(512) void gla_chunk_state_kernel(GlaArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int h = blockIdx.x, ch = blockIdx.y, tid = threadIdx.x, NT = blockDim.x;
+    const int wv = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
+    const int n = a.n, p = a.p, N = pad16(n), P = pad16(p), SP = P + 4, nt = N / 16, pt = P / 16;
     const int start = a.ch_start[ch], len = a.ch_len[ch];
-    const int64_t unit = (int64_t)ch * a.H + h, c = (int64_t)h * a.n + (i < a.n ? i : a.n - 1);
-    const float bias = a.bias ? a.bias[c] : 0.f;
-    float4* kt = reinterpret_cast<float4*>(a.kt + unit * (kGCh * N)) + (int64_t)(i >> 4) * 256 + (i & 15);
-    float suf = 1.f;
-#pragma unroll
-    for (int blk = 3; blk >= 0; --blk) {
+    const int64_t unit = (int64_t)ch * a.H + h;
+    if (a.vec_v) {
+        const int p4 = P / 4;
+        for (int i = tid; i < kGCh * p4; i += NT) {
+            const int t = i / p4, c = 4 * (i - t * p4);
+            float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (t < len && c < p) v = *reinterpret_cast<const float4*>(a.v + (int64_t)(start + t) * a.ldv + (int64_t)h * p + c);
+            *reinterpret_cast<float4*>(lds + t * SP + c) = v;
+        }
+    } else {
+        for (int i = tid; i < kGCh * P; i += NT) {
+            const int t = i / P, c = i - t * P;
+            lds[t * SP + c] = (t < len && c < p) ? a.v[(int64_t)(start + t) * a.ldv + (int64_t)h * p + c] : 0.f;
+        }
+    }
+    float w[4][4], run = 1.f;
+    auto keys = [&](int it) {
+        const int i = 16 * it + r;
+        const int64_t c = (int64_t)h * n + (i < n ? i : n - 1);
+        const float bias = a.bias ? a.bias[c] : 0.f;
         float kk[16], zz[16];
 #pragma unroll
-        for (int t = 0; t < 16; ++t) {
-            const int tt = 16 * blk + t;
-            const int64_t tok = start + (tt < len ? tt : len - 1);
-            kk[t] = a.k[tok * a.ldk + c];
-            zz[t] = a.z[tok * a.ldz + c];
+        for (int e = 0; e < 16; ++e) {
+            const int t = 16 * (e >> 2) + 4 * g + (e & 3);
+            const int64_t tok = start + (t < len ? t : len - 1);
+            kk[e] = a.k[tok * a.ldk + c];
+            zz[e] = a.z[tok * a.ldz + c];
         }
+        run = 1.f;                           // product of the gates of the blocks behind
 #pragma unroll
-        for (int g = 3; g >= 0; --g) {
-            float o[4];
+        for (int blk = 3; blk >= 0; --blk) {
+            float al[4], mine = 1.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const bool ok = i < n && 16 * blk + 4 * g + j < len;
+                al[j] = ok ? gla_decay(a, zz[4 * blk + j], bias) : 1.f;
+                w[blk][j] = ok ? kk[4 * blk + j] : 0.f;
+                mine *= al[j];
+            }
+            const float p1 = __shfl(mine, (lane + 16) & 63, 64), p2 = __shfl(mine, (lane + 32) & 63, 64);
+            const float p3 = __shfl(mine, (lane + 48) & 63, 64);
+            float suf = run;
+            if (g < 3) suf *= p1;
+            if (g < 2) suf *= p2;
+            if (g < 1) suf *= p3;
 #pragma unroll
             for (int j = 3; j >= 0; --j) {
-                const int t = 4 * g + j;
-                const bool ok = i < a.n && 16 * blk + t < len;
-                o[j] = ok ? kk[t] * suf : 0.f;
-                suf *= ok ? gla_decay(a, zz[t], bias) : 1.f;
+                w[blk][j] *= suf;
+                suf *= al[j];
             }
-            kt[blk * 64 + g * 16] = make_float4(o[0], o[1], o[2], o[3]);
+            run *= ((mine * p1) * p2) * p3;
+        }
+    };
+    keys(wv < nt ? wv : 0);
+    __syncthreads();
+    for (int it = wv; it < nt; it += NT / 64) {
+        if (it != wv) keys(it);
+        if (g == 0) a.gc[unit * N + 16 * it + r] = run;
+        float4* out = reinterpret_cast<float4*>(a.s0 + unit * ((int64_t)N * P)) + it * pt * 64 + lane;
+        for (int ct = 0; ct < pt; ++ct) {
+            const float* v = lds + 4 * g * SP + 16 * ct + r;
+            f32x4_t y0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, y1 = y0;      // neighbouring products do not wait for each other
+#pragma unroll
+            for (int blk = 0; blk < 4; ++blk) {
+                MV_DMFMA(y0, w[blk][0], v[16 * blk * SP]);
+                MV_DMFMA(y1, w[blk][1], v[(16 * blk + 1) * SP]);
+                MV_DMFMA(y0, w[blk][2], v[(16 * blk + 2) * SP]);
+                MV_DMFMA(y1, w[blk][3], v[(16 * blk + 3) * SP]);
+            }
+            y0 += y1;
+            out[ct * 64] = make_float4(y0[0], y0[1], y0[2], y0[3]);
         }
     }
-    a.gc[unit * N + i] = suf;
 }
 
-// One wave per (row, head, 16 state rows, 16 columns): lane (r, g) holds rows 4 g .. + 3 of column r.  The state each chunk
-// starts from goes to s0, tile by tile in the order the out kernel's lanes read it.  The waves of a workgroup share their
-// columns (and thereby the values they read), nothing else.
+// Four state values a thread, in the tiles' order: the state each chunk starts from takes the place of what it adds.
 __global__ __launch_bounds__(256) void gla_chunk_carry_kernel(GlaArgs a) {
-    const int h = blockIdx.x, b = blockIdx.z, nch = a.row_nch[b];
-    const int wv = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
-    const int n = a.n, p = a.p, N = pad16(n), P = pad16(p), nt = N / 16, pt = P / 16;
-    const int ct = blockIdx.y % pt, it = (blockIdx.y / pt) * 4 + wv;
-    if (nch == 0 || it >= nt) return;
-    const int col = 16 * ct + r;
-    const bool vc = col < p, carried = a.row_ctx[b] > 0;
-    const int first = a.row_start[b], total = a.row_len[b];
-    float* st = a.state + ((int64_t)a.row_slot[b] * a.H + h) * n * p + col;
-    f32x4_t S;
+    const int h = blockIdx.y, b = blockIdx.z, nch = a.row_nch[b], e = blockIdx.x * 256 + threadIdx.x;
+    const int n = a.n, p = a.p, N = pad16(n), P = pad16(p), pt = P / 16;
+    if (nch == 0 || e >= N * P / 4) return;
+    const int tile = e >> 6, it = tile / pt, g = (e >> 4) & 3, row = 16 * it + 4 * g, col = 16 * (tile - it * pt) + (e & 15);
+    const bool carried = a.row_ctx[b] > 0;
+    float* st = a.state + (((int64_t)a.row_slot[b] * a.H + h) * n + row) * p + col;
+    float S[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        const int i = 16 * it + 4 * g + j;
-        S[j] = (carried && vc && i < n) ? st[(int64_t)i * p] : 0.f;
-    }
+    for (int j = 0; j < 4; ++j) S[j] = (carried && col < p && row + j < n) ? st[(int64_t)j * p] : 0.f;
     const int64_t u0 = (int64_t)a.row_ch0[b] * a.H + h;
-    const float* vp = a.v + (int64_t)h * p + (vc ? col : p - 1);
-    struct Operands {
-        float4 kt[4], gm;
-        float v[16];
-    };
-    auto fetch = [&](int c, Operands& x) {
-        const int64_t unit = u0 + (int64_t)c * a.H;
-        const float4* k = reinterpret_cast<const float4*>(a.kt + unit * (kGCh * N)) + it * 256 + lane;
+    constexpr int kB = 4;                    // chunks whose values are requested together
+    for (int c0 = 0; c0 < nch; c0 += kB) {
+        float4 d[kB], gm[kB];
 #pragma unroll
-        for (int t = 0; t < 4; ++t) x.kt[t] = k[64 * t];
-        x.gm = *reinterpret_cast<const float4*>(a.gc + unit * N + 16 * it + 4 * g);
-        const int t0 = kGCh * c, left = total - t0;
-#pragma unroll
-        for (int i = 0; i < 16; ++i) {
-            const int t = 16 * (i >> 2) + 4 * g + (i & 3);
-            x.v[i] = vp[(int64_t)(first + t0 + (t < left ? t : left - 1)) * a.ldv];
+        for (int u = 0; u < kB; ++u) {
+            const int64_t unit = u0 + (int64_t)(c0 + u < nch ? c0 + u : nch - 1) * a.H;
+            d[u] = reinterpret_cast<const float4*>(a.s0 + unit * ((int64_t)N * P))[e];
+            gm[u] = *reinterpret_cast<const float4*>(a.gc + unit * N + row);
         }
-    };
-    auto body = [&](Operands& cur, int c) {
-        float4* s0 = reinterpret_cast<float4*>(a.s0 + (u0 + (int64_t)c * a.H) * ((int64_t)N * P)) + (it * pt + ct) * 64 + lane;
-        *s0 = make_float4(S[0], S[1], S[2], S[3]);      // what this chunk starts from
-        // two accumulators: neighbouring products do not wait for each other
-        f32x4_t y0 = f32x4_t{S[0] * cur.gm.x, S[1] * cur.gm.y, S[2] * cur.gm.z, S[3] * cur.gm.w};
-        f32x4_t y1 = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            MV_DMFMA(y0, cur.kt[t].x, vc ? cur.v[4 * t] : 0.f);
-            MV_DMFMA(y1, cur.kt[t].y, vc ? cur.v[4 * t + 1] : 0.f);
-            MV_DMFMA(y0, cur.kt[t].z, vc ? cur.v[4 * t + 2] : 0.f);
-            MV_DMFMA(y1, cur.kt[t].w, vc ? cur.v[4 * t + 3] : 0.f);
+        for (int u = 0; u < kB; ++u) {
+            if (c0 + u >= nch) break;
+            const int64_t unit = u0 + (int64_t)(c0 + u) * a.H;
+            reinterpret_cast<float4*>(a.s0 + unit * ((int64_t)N * P))[e] = make_float4(S[0], S[1], S[2], S[3]);
+            S[0] = fmaf(gm[u].x, S[0], d[u].x);
+            S[1] = fmaf(gm[u].y, S[1], d[u].y);
+            S[2] = fmaf(gm[u].z, S[2], d[u].z);
+            S[3] = fmaf(gm[u].w, S[3], d[u].w);
         }
-        S = y0 + y1;
-        if (c + 3 < nch) fetch(c + 3, cur);
-    };
-    // three sets of operands: a chunk's are requested while the two before it are worked on
-    Operands x0, x1, x2;
-    fetch(0, x0);
-    if (nch > 1) fetch(1, x1);
-    if (nch > 2) fetch(2, x2);
-    for (int c = 0; c < nch; c += 3) {
-        body(x0, c);
-        if (c + 1 < nch) body(x1, c + 1);
-        if (c + 2 < nch) body(x2, c + 2);
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        const int i = 16 * it + 4 * g + j;
-        if (vc && i < n) st[(int64_t)i * p] = S[j];
-    }
+    for (int j = 0; j < 4; ++j)
+        if (col < p && row + j < n) st[(int64_t)j * p] = S[j];
 }
 
 // One workgroup per (head, chunk), eight waves.  NM: groups of 32 state rows (n <= 32 NM); CTW: 16-column tiles a wave owns.
@@ -520,7 +534,7 @@ int mv_gated_linear_chunked_ok(int n, int p) {
 
 int64_t mv_gated_linear_scratch_floats(int n, int p) {
     const int64_t N = (n + 15) & ~15, P = (p + 15) & ~15;
-    return mv::kGCh * N + N * P + N;
+    return N * P + N;
 }
 
 int mv_gated_linear_attn(const float* q, int64_t ldq, const float* k, int64_t ldk, const float* v, int64_t ldv,
@@ -551,6 +565,7 @@ int mv_gated_linear_attn(const float* q, int64_t ldq, const float* k, int64_t ld
     a.ch_start = ch_start; a.ch_len = ch_len; a.row_ch0 = row_ch0; a.row_nch = row_nch;
     a.vec_in = n % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && ldz % 4 == 0 && aligned16(q) && aligned16(k) && aligned16(z) &&
                (!z_bias || aligned16(z_bias));
+    a.vec_v = p % 4 == 0 && ldv % 4 == 0 && aligned16(v);
     a.vec_out = p % 16 == 0 && ldg % 4 == 0 && ldo % 4 == 0 && aligned16(gate) && aligned16(out) && aligned16(norm);
     hipStream_t s = (hipStream_t)stream;
     if (chunks == 0 || short_tokens != 0) {
@@ -576,12 +591,13 @@ int mv_gated_linear_attn(const float* q, int64_t ldq, const float* k, int64_t ld
     }
     if (chunks > 0) {
         const int64_t N = (n + 15) & ~15, P = (p + 15) & ~15, U = (int64_t)chunks * heads;
-        a.kt = scratch;
-        a.s0 = a.kt + U * kGCh * N;
+        a.s0 = scratch;
         a.gc = a.s0 + U * N * P;
-        hipLaunchKernelGGL(gla_chunk_keys_kernel, dim3((unsigned)((heads * N + 255) / 256), chunks), dim3(256), 0, s, a);
-        const dim3 gc(heads, (unsigned)((P / 16) * ((N / 16 + 3) / 4)), rows);
-        hipLaunchKernelGGL(gla_chunk_carry_kernel, gc, dim3(256), 0, s, a);
+        const size_t lds0 = (size_t)kGCh * (P + 4) * sizeof(float);
+        static LdsOptIn opt0;
+        if (int rc = ensure_dynamic_lds((const void*)gla_chunk_state_kernel, lds0, opt0)) return rc;
+        hipLaunchKernelGGL(gla_chunk_state_kernel, dim3(heads, chunks), dim3(N > 64 ? 512 : 256), lds0, s, a);
+        hipLaunchKernelGGL(gla_chunk_carry_kernel, dim3((unsigned)((N * P / 4 + 255) / 256), heads, rows), dim3(256), 0, s, a);
         const size_t lds = gla_out_lds(n);
         static LdsOptIn opt[2][3][2];
         const dim3 go(heads, chunks);

@@ -141,35 +141,11 @@ __global__ __launch_bounds__(256) void moe_route_scored_kernel(const void* h_, i
     }
 }
 
-// One workgroup per token; the choice is one wave's: a lane per group of experts, then a lane per expert in turns.
-template <bool F32>
-__global__ __launch_bounds__(256) void moe_route_grouped_kernel(const void* h_, int64_t ldh, const float* wr,
-                                                                const float* correction, int* ids, float* wts, int n,
-                                                                int E, int groups, int keep, int top) {
-    __shared__ float sc[kMaxExperts], ch[kMaxExperts], worth[kMaxExperts];
-    const int t = blockIdx.x, wv = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    for (int e = wv; e < E; e += 4) {
-        const float* w = wr + (int64_t)e * n;
-        float dot = 0.f;
-        if (F32) {
-            const float* h = (const float*)h_ + (int64_t)t * ldh;
-#pragma unroll 8
-            for (int c = lane; c < n; c += 64) dot = fmaf(h[c], w[c], dot);
-        } else {
-            const uint16_t* h = (const uint16_t*)h_ + (int64_t)t * ldh;
-#pragma unroll 8
-            for (int c = lane; c < n; c += 64) dot = fmaf(bf16_bits_to_f32(h[c]), w[c], dot);
-        }
-        dot = wave_sum(dot);
-        if (lane == 0) {
-            const float s = 1.0f / (1.0f + expf(-dot));
-            sc[e] = s;
-            ch[e] = correction ? s + correction[e] : s;
-        }
-    }
-    __syncthreads();
+// The group-limited choice of one token, by one wave: sc = scores, ch = choice scores (spoilt), worth = a place per group.
+__device__ __forceinline__ void choose_grouped(const float* sc, float* ch, float* worth, int lane, int E, int groups, int keep,
+                                               int top, int* ids, float* wts) {
     const int per = E / groups;
-    for (int g = threadIdx.x; g < groups; g += 256) {
+    for (int g = lane; g < groups; g += 64) {
         float a = -INFINITY, b = -INFINITY;          // the two largest
         for (int i = 0; i < per; ++i) {
             const float v = ch[g * per + i];
@@ -182,16 +158,15 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const void* h_, 
         }
         worth[g] = per > 1 ? a + b : a;
     }
-    __syncthreads();
+    __builtin_amdgcn_wave_barrier();
     // a group that `keep` others are ahead of is out: its experts can no longer be chosen, whatever their scores
-    for (int g = threadIdx.x; g < groups; g += 256) {
+    for (int g = lane; g < groups; g += 64) {
         int ahead = 0;
         for (int o = 0; o < groups; ++o) ahead += worth[o] > worth[g] || (worth[o] == worth[g] && o < g);
         if (ahead >= keep)
             for (int i = 0; i < per; ++i) ch[g * per + i] = -INFINITY;
     }
-    __syncthreads();
-    if (wv > 0) return;
+    __builtin_amdgcn_wave_barrier();
     for (int k = 0; k < top; ++k) {
         float bv = -INFINITY;
         int best = E;
@@ -211,11 +186,114 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const void* h_, 
         }
         best = best < E ? best : E - 1;              // scores that are not numbers choose nothing: stay in bounds
         if (lane == 0) {
-            ids[(int64_t)t * top + k] = best;
-            wts[(int64_t)t * top + k] = sc[best];
+            ids[k] = best;
+            wts[k] = sc[best];
             ch[best] = -INFINITY;
         }
         __builtin_amdgcn_wave_barrier();
+    }
+}
+
+// One workgroup per token, a wave per expert in turns.  `vec`: rows in 16-byte pieces (n a multiple of 8, aligned).
+template <bool F32>
+__global__ __launch_bounds__(1024) void moe_route_grouped_kernel(const void* h_, int64_t ldh, const float* wr,
+                                                                 const float* correction, int* ids, float* wts, int n,
+                                                                 int E, int groups, int keep, int top, int vec) {
+    extern __shared__ float lds[];
+    float* sc = lds;                     // scores | choice scores | what each group is worth
+    const int t = blockIdx.x, wv = threadIdx.x >> 6, lane = threadIdx.x & 63, NW = blockDim.x >> 6;
+    const float* hf = (const float*)h_ + (int64_t)t * ldh;
+    const uint16_t* hb = (const uint16_t*)h_ + (int64_t)t * ldh;
+    for (int e = wv; e < E; e += NW) {
+        const float* w = wr + (int64_t)e * n;
+        float dot = 0.f;
+        if (vec) {
+#pragma unroll 2
+            for (int c = 8 * lane; c < n; c += 512) {
+                const float4 wa = *reinterpret_cast<const float4*>(w + c), wb = *reinterpret_cast<const float4*>(w + c + 4);
+                float x[8];
+                if (F32) {
+                    const float4 a = *reinterpret_cast<const float4*>(hf + c), b = *reinterpret_cast<const float4*>(hf + c + 4);
+                    x[0] = a.x; x[1] = a.y; x[2] = a.z; x[3] = a.w; x[4] = b.x; x[5] = b.y; x[6] = b.z; x[7] = b.w;
+                } else {
+                    const uint4 a = ld16(hb + c);
+                    x[0] = bf16_lo(a.x); x[1] = bf16_hi(a.x); x[2] = bf16_lo(a.y); x[3] = bf16_hi(a.y);
+                    x[4] = bf16_lo(a.z); x[5] = bf16_hi(a.z); x[6] = bf16_lo(a.w); x[7] = bf16_hi(a.w);
+                }
+                dot = fmaf(x[0], wa.x, fmaf(x[1], wa.y, fmaf(x[2], wa.z, fmaf(x[3], wa.w, dot))));
+                dot = fmaf(x[4], wb.x, fmaf(x[5], wb.y, fmaf(x[6], wb.z, fmaf(x[7], wb.w, dot))));
+            }
+        } else {
+            for (int c = lane; c < n; c += 64) dot = fmaf(F32 ? hf[c] : bf16_bits_to_f32(hb[c]), w[c], dot);
+        }
+        dot = wave_sum(dot);
+        if (lane == 0) {
+            const float s = 1.0f / (1.0f + expf(-dot));
+            sc[e] = s;
+            sc[E + e] = correction ? s + correction[e] : s;
+        }
+    }
+    __syncthreads();
+    if (wv == 0)
+        choose_grouped(sc, sc + E, sc + 2 * E, lane, E, groups, keep, top, ids + (int64_t)t * top, wts + (int64_t)t * top);
+}
+
+// The same for steps of many tokens: a workgroup per 16 tokens, the logits as 16 experts x 16 tokens on
+// v_mfma_f32_16x16x4_f32 (true fp32), eight waves sharing the contraction.  n a multiple of 16, rows aligned for pieces of
+// four values, E <= kRouteTileE.
+constexpr int kRouteTileE = 256;
+
+template <bool F32>
+__global__ __launch_bounds__(512) void moe_route_grouped_tile_kernel(const void* h_, int64_t ldh, const float* wr,
+                                                                     const float* correction, int* ids, float* wts, int T,
+                                                                     int n, int E, int groups, int keep, int top) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    float* part = lds;                   // [8 waves][16 tokens][16 experts]
+    float* sc = lds + 8 * 256;           // [16 tokens][scores | choice scores | what each group is worth]
+    const int per_tok = 2 * E + groups;
+    const int t0 = blockIdx.x * 16, wv = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
+    const int tn = T - t0 < 16 ? T - t0 : 16;
+    const int64_t row = (int64_t)(t0 + (r < tn ? r : 0)) * ldh;
+    const float* hf = (const float*)h_ + row;
+    const uint16_t* hb = (const uint16_t*)h_ + row;
+    for (int e0 = 0; e0 < E; e0 += 16) {
+        const float* w = wr + (int64_t)(e0 + r < E ? e0 + r : e0) * n;
+        f32x4_t a0 = f32x4_t{0.f, 0.f, 0.f, 0.f}, a1 = a0;
+#pragma unroll 4
+        for (int c = 16 * wv + 4 * g; c < n; c += 128) {
+            const float4 wc = *reinterpret_cast<const float4*>(w + c);
+            float4 x;
+            if (F32) {
+                x = *reinterpret_cast<const float4*>(hf + c);
+            } else {
+                const uint2 b = *reinterpret_cast<const uint2*>(hb + c);
+                x = make_float4(bf16_lo(b.x), bf16_hi(b.x), bf16_lo(b.y), bf16_hi(b.y));
+            }
+            a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(wc.x, x.x, a0, 0, 0, 0);
+            a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(wc.y, x.y, a1, 0, 0, 0);
+            a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(wc.z, x.z, a0, 0, 0, 0);
+            a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(wc.w, x.w, a1, 0, 0, 0);
+        }
+        a0 += a1;                        // lane (r, g): experts e0 + 4 g .. + 3 of token r
+        *reinterpret_cast<float4*>(part + wv * 256 + r * 16 + 4 * g) = make_float4(a0[0], a0[1], a0[2], a0[3]);
+        __syncthreads();
+        if (threadIdx.x < 256) {
+            float z = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) z += part[i * 256 + threadIdx.x];
+            const int e = e0 + (threadIdx.x & 15);
+            if (e < E) {
+                float* s = sc + (threadIdx.x >> 4) * per_tok;
+                const float v = 1.0f / (1.0f + expf(-z));
+                s[e] = v;
+                s[E + e] = correction ? v + correction[e] : v;
+            }
+        }
+        __syncthreads();
+    }
+    for (int u = wv; u < tn; u += 8) {
+        float* s = sc + u * per_tok;
+        choose_grouped(s, s + E, s + 2 * E, lane, E, groups, keep, top, ids + (int64_t)(t0 + u) * top, wts + (int64_t)(t0 + u) * top);
     }
 }
 
@@ -354,8 +432,19 @@ int mv_moe_route_grouped(const void* h, int64_t ldh, const float* w_router, cons
     if (tokens == 0) return MV_OK;
     if (!h || !w_router || !ids || !weights || ldh < n) return MV_ERR_INVALID_ARG;
     hipStream_t s = (hipStream_t)stream;
-    if (f32) hipLaunchKernelGGL(moe_route_grouped_kernel<true>, dim3(tokens), dim3(256), 0, s, h, ldh, w_router, correction, ids, weights, n, experts, groups, keep, top);
-    else hipLaunchKernelGGL(moe_route_grouped_kernel<false>, dim3(tokens), dim3(256), 0, s, h, ldh, w_router, correction, ids, weights, n, experts, groups, keep, top);
+    if (tokens > 64 && experts <= kRouteTileE && n % 16 == 0 && ldh % 4 == 0 && aligned16(h) && aligned16(w_router)) {
+        const size_t lds = (8 * 256 + (size_t)16 * (2 * experts + groups)) * sizeof(float);
+        const dim3 tiles((tokens + 15) / 16);
+        if (f32) hipLaunchKernelGGL(moe_route_grouped_tile_kernel<true>, tiles, dim3(512), lds, s, h, ldh, w_router, correction, ids, weights, tokens, n, experts, groups, keep, top);
+        else hipLaunchKernelGGL(moe_route_grouped_tile_kernel<false>, tiles, dim3(512), lds, s, h, ldh, w_router, correction, ids, weights, tokens, n, experts, groups, keep, top);
+        return check_launch();
+    }
+    const int vec = n % 8 == 0 && ldh % 8 == 0 && aligned16(h) && aligned16(w_router);
+    int nt = 256;
+    while (nt < 1024 && nt / 64 < experts) nt *= 2;
+    const size_t lds = (size_t)(2 * experts + groups) * sizeof(float);
+    if (f32) hipLaunchKernelGGL(moe_route_grouped_kernel<true>, dim3(tokens), dim3(nt), lds, s, h, ldh, w_router, correction, ids, weights, n, experts, groups, keep, top, vec);
+    else hipLaunchKernelGGL(moe_route_grouped_kernel<false>, dim3(tokens), dim3(nt), lds, s, h, ldh, w_router, correction, ids, weights, n, experts, groups, keep, top, vec);
     return check_launch();
 }
 

@@ -837,27 +837,40 @@ __global__ __launch_bounds__(256) void qkv_headnorm_rotary_store_kernel(float* q
             }
         }
     }
+    // a head's values and biases, requested while the head before it is worked on
+    float n0[NI], n1[NI], m0[NI], m1[NI];
+    auto fetch = [&](int u) {
+        if (u >= u1 || u >= H + G) return;
+        const float* x = row + (int64_t)u * d;       // q's heads, then k's
+        const float* b = u < H ? (qb ? qb + (int64_t)u * d : nullptr) : (kb ? kb + (int64_t)(u - H) * d : nullptr);
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int j = lane + 64 * i;
+            n0[i] = n1[i] = m0[i] = m1[i] = 0.f;
+            if (j >= items) continue;
+            const int a0 = j < half ? (adjacent ? 2 * j : j) : half + j, a1 = adjacent ? 2 * j + 1 : j + half;
+            n0[i] = x[a0];
+            if (b) m0[i] = b[a0];
+            if (j < half) {
+                n1[i] = x[a1];
+                if (b) m1[i] = b[a1];
+            }
+        }
+    };
+    fetch(u0);
     for (int u = u0; u < u1; ++u) {
         if (u < H + G) {
             const bool isq = u < H;
-            float* x = row + (isq ? (int64_t)u * d : (int64_t)H * d + (int64_t)(u - H) * d);
-            const float* b = isq ? (qb ? qb + (int64_t)u * d : nullptr) : (kb ? kb + (int64_t)(u - H) * d : nullptr);
+            float* x = row + (int64_t)u * d;
             const float* w = isq ? qn : kn;
             float x0[NI], x1[NI], ss = 0.f;
 #pragma unroll
             for (int i = 0; i < NI; ++i) {
-                const int j = lane + 64 * i;
-                x0[i] = x1[i] = 0.f;
-                if (j >= items) continue;
-                const int a0 = j < half ? (adjacent ? 2 * j : j) : half + j;
-                x0[i] = b ? x[a0] + b[a0] : x[a0];
-                ss += x0[i] * x0[i];
-                if (j < half) {
-                    const int a1 = adjacent ? 2 * j + 1 : j + half;
-                    x1[i] = b ? x[a1] + b[a1] : x[a1];
-                    ss += x1[i] * x1[i];
-                }
+                x0[i] = n0[i] + m0[i];
+                x1[i] = n1[i] + m1[i];
+                ss += x0[i] * x0[i] + x1[i] * x1[i];
             }
+            fetch(u + 1);
             float inv = 1.f;
             if (w) inv = 1.0f / sqrtf(wave_sum(ss) / (float)d + eps);
             T_* dst = kc + (slot + (u - H)) * d;

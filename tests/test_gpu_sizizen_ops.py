@@ -456,7 +456,8 @@ def test_arguments_outside_the_kernels_limits_are_refused(ops):
 # ----------------------------------------------------------------------------------------------- routed experts
 @pytest.mark.parametrize("f32", [False, True])
 @pytest.mark.parametrize("T,E,groups,keep,top,W", [(37, 12, 3, 2, 4, 96), (5, 8, 8, 2, 2, 40), (3, 6, 1, 1, 6, 33), (130, 40, 4, 1, 6, 96),
-                                                   (9, 96, 12, 5, 16, 200), (2, 1, 1, 1, 1, 24), (1, 256, 8, 4, 8, 512)])
+                                                   (9, 96, 12, 5, 16, 200), (2, 1, 1, 1, 1, 24), (1, 256, 8, 4, 8, 512), (83, 100, 10, 3, 8, 208),
+                                                   (65, 16, 4, 2, 4, 1024), (70, 256, 8, 4, 8, 48), (66, 300, 3, 1, 5, 64)])
 @pytest.mark.parametrize("corrected", [True, False])
 def test_group_limited_choice(ops, f32, T, E, groups, keep, top, W, corrected):
     g = torch.Generator().manual_seed(E + top)
