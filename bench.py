@@ -818,8 +818,9 @@ def sizizen_compare(args, dev):
     dense feed-forwards (gate, up, down of 4 x width), once with every one routed (16 experts in four groups of which two
     are kept, four experts used, beside a shared one: up and down of 6 x width active) - beside Pagazen and Fagunex, all
     through InferenceEngine.run_ragged.  Random weights, 4 layers, vocabulary 32000, 128-wide heads, a low-rank map of 128.
-    Pagazen: a parallel mixer in every layer with the same heads, a window as long as Sizizen's chunks (1024), the same
-    128 x 128 states, up and down with 6 x width; Fagunex: three gated recurrences and one latent attention, routed
+    Chunks of a little more than half of --ctx (1088 of 2048), so that a decoded token sees nearly a whole one.  Pagazen: a
+    parallel mixer in every layer with the same heads, a window of 1024, the same 128 x 128 states, up and down with 6 x
+    width; Fagunex: three gated recurrences and one latent attention, routed
     experts with gate, up and down of 4 x width active."""
     import micro_vllm_amd  # noqa: F401
     from micro_vllm_amd.core.engine import InferenceEngine
@@ -832,12 +833,14 @@ def sizizen_compare(args, dev):
         return pagazen.build_random_model(cfg, 1)
 
     S, layers, rows = args.ctx, 4, []
+    chunk = max(1, S // 2 + S // 32)
     for width in [int(w) for w in args.sizizen_widths.split(",")]:
         row = {"width": width, "layers": layers, "ctx": S}
-        for name, make in (("sizizen_dense", lambda: sizizen.build_random_model(sizizen.bench_config(width, layers), 1, rank=128)),
+        for name, make in (("sizizen_dense", lambda: sizizen.build_random_model(
+                               sizizen.bench_config(width, layers, chunk=chunk), 1, rank=128)),
                            ("pagazen", lambda: pagazen_parallel(width)),
                            ("sizizen_routed", lambda: sizizen.build_random_model(
-                               sizizen.bench_config(width, layers, ff_mult=6, moe_every=1), 1, rank=128)),
+                               sizizen.bench_config(width, layers, ff_mult=6, moe_every=1, chunk=chunk), 1, rank=128)),
                            ("fagunex", lambda: fagunex.build_random_model(fagunex.bench_config(width, layers), 1))):
             model = make()
             eng = InferenceEngine(model=model, max_batch_size=8, max_prefill_tokens=S, n_blocks=9 * (S // 64 + 4),

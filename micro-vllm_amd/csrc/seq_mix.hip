@@ -1405,7 +1405,11 @@ __global__ __launch_bounds__(256) void window_attn_tile_kernel(const float* q, i
     // values as pairs of neighbouring keys: dword [i][c] = V[2i][c] | V[2i+1][c] << 16, which is how the matrix
     // instruction wants them (two contraction slots per register)
     __shared__ __attribute__((aligned(16))) uint32_t Vp[32][SV];
-    const int ch = blockIdx.x, h = blockIdx.y, g = h / (H / G);
+    // Workgroups 256 apart share a compute unit; a chunk's place decides how many keys it reads.  The chunks of later heads
+    // are taken in a rotated order, so that a unit gets chunks of unequal places.
+    const int h = blockIdx.y, g = h / (H / G), nch = gridDim.x;
+    const int rounds = (nch * (int)gridDim.y + 255) >> 8, turn = ((h * nch) >> 8) * (nch / rounds);
+    const int ch = (int)((blockIdx.x + turn) % nch);
     const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, r = lane & 15, qd = lane >> 4;
     const int start = ch_start[ch], len = ch_len[ch];
     const int* bt = pr.block_table + (int64_t)pr.tok_row[start] * pr.bt_stride;
