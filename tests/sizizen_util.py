@@ -48,7 +48,7 @@ def config_b():
     projections and the matrix-core attention take (so the bf16 run uses both)."""
     return SizizenConfig(vocab_size=256, width=128, eps=1e-6, layers=[
         layer(attention(heads=2, kv_heads=2, dim=64, vdim=64, chunk=128, rot=64, base=100.0, scale=0.125), linear(heads=2, dim=64, vdim=64, tau=1.0), dense(128)),
-        layer(attention(heads=4, kv_heads=1, dim=64, vdim=32, chunk=64, rot=16, scale=0.2), linear(heads=1, dim=128, vdim=128, tau=16.0),
+        layer(attention(heads=6, kv_heads=2, dim=64, vdim=32, chunk=64, rot=32, scale=0.2), linear(heads=1, dim=128, vdim=128, tau=16.0),
               moe(experts=4, groups=1, keep=1, top=1, ff=64, shared=64)),
         layer(attention(heads=1, kv_heads=1, dim=32, vdim=32, chunk=1, rot=32, scale=0.2), linear(heads=4, dim=16, vdim=32, tau=2.0),
               moe(experts=6, groups=6, keep=6, top=6, ff=128, shared=0)),

@@ -255,7 +255,7 @@ def attend(ops, q, k, v, H, G, d, dv, scale, chunk, portions, f32=True, tiled=Tr
     return torch.cat(out)
 
 
-@pytest.mark.parametrize("H,G,d,dv,chunk", [(6, 2, 40, 24, 37), (4, 1, 64, 64, 65), (2, 2, 128, 64, 300), (9, 1, 32, 32, 64), (4, 1, 64, 32, 64),
+@pytest.mark.parametrize("H,G,d,dv,chunk", [(6, 2, 40, 24, 37), (4, 1, 64, 64, 65), (2, 2, 128, 64, 300), (9, 1, 32, 32, 64), (6, 2, 64, 32, 64),
                                             (2, 1, 64, 32, 100), (3, 3, 8, 8, 1), (2, 1, 96, 96, 17)])
 def test_attention_within_chunks(ops, H, G, d, dv, chunk):
     """All four forms (one workgroup per head, shared reads, shared reads cut into pieces, matrix cores), whole prompts,
